@@ -6,6 +6,7 @@ from . import lerazen as _lerazen  # registers "Lerazen"
 from . import nasedra as _nasedra  # registers "Nasedra"
 from . import dikolix as _dikolix  # registers "Dikolix"
 from . import vagelix as _vagelix  # registers "Vagelix"
+from . import begasun as _begasun  # registers "Begasun"
 from .engine_args import EngineArgs
 
 __all__ = ["ConfigError", "Qwen2Config", "read_config_json", "Architecture", "known_architectures",

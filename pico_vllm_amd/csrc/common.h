@@ -50,6 +50,12 @@ template <typename T> __device__ __forceinline__ void store_f32(T* p, float v);
 template <> __device__ __forceinline__ void store_f32<float>(float* p, float v) { *p = v; }
 template <> __device__ __forceinline__ void store_f32<bf16_t>(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 
+// 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), written with (1 + tanh(a)) / 2 = 1 / (1 + exp(-2 a))
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  const float a = 0.7978845608028654f * fmaf(0.044715f * z * z, z, z);
+  return z / (1.0f + expf(-2.0f * a));
+}
+
 // A value combined with the one 16 (32) lanes across, in both lanes: one vector instruction of gfx950
 // (v_permlane16_swap / v_permlane32_swap give both values in two registers) where an exchange through the LDS crossbar
 // (what __shfl_xor compiles to) waits in line behind the tiles' reads.  Maximum and sum are symmetric, so both lanes

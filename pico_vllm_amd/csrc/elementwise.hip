@@ -293,19 +293,34 @@ extern "C" int pico_residual_add(float* resid, const void* delta, int delta_dtyp
 // SwiGLU: out[t, i] = silu(gu[t, i]) * gu[t, I + i], silu(g) = g * sigmoid(g)
 // (pico_vllm/kernels/swiglu.py:22-41: gate is the first half of the last dim).
 // ---------------------------------------------------------------------------
-template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total) {
+// The activations of a pair (gate, up): ACT_SWIGLU silu(g) u;  ACT_CLIPPED g' sigmoid(alpha g') (u' + 1) with g' = min(g, limit)
+// and u' = u clamped to -limit .. limit.
+#define ACT_SWIGLU 0
+#define ACT_CLIPPED 1
+template <int ACT>
+__device__ __forceinline__ float gated_act(float g, float u, float limit, float alpha) {
+  if (ACT == ACT_CLIPPED) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+  }
+  return g / (1.0f + expf(-g)) * u;
+}
+
+template <typename T, int ACT>
+__global__ void gated_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total, float limit, float alpha) {
   size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const size_t row = idx / I, col = idx % I;
   const float g = load_f32(gu + row * 2 * (size_t)I + col);
   const float u = load_f32(gu + row * 2 * (size_t)I + I + col);
-  const float s = g / (1.0f + expf(-g));
-  store_f32(out + idx, s * u);
+  store_f32(out + idx, gated_act<ACT>(g, u, limit, alpha));
 }
 
 // bfloat16 rows whose halves start on 16 bytes (I % 8 == 0): eight elements per thread, 16-byte loads and stores
-__global__ void swiglu_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out, int I8, size_t total8) {
+template <int ACT>
+__global__ void gated_act_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out, int I8, size_t total8, float limit,
+                                        float alpha) {
   typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total8) return;
@@ -317,28 +332,68 @@ __global__ void swiglu_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __re
   for (int i = 0; i < 4; i++) {
     const float g0 = __uint_as_float(g[i] << 16), g1 = __uint_as_float(g[i] & 0xffff0000u);
     const float u0 = __uint_as_float(u[i] << 16), u1 = __uint_as_float(u[i] & 0xffff0000u);
-    o[i] = pack2_bf16(g0 / (1.0f + expf(-g0)) * u0, g1 / (1.0f + expf(-g1)) * u1);
+    o[i] = pack2_bf16(gated_act<ACT>(g0, u0, limit, alpha), gated_act<ACT>(g1, u1, limit, alpha));
   }
   *reinterpret_cast<u32x4*>(out + idx * 8) = o;
 }
 
-extern "C" int pico_swiglu(const void* gu, void* out, int dtype, int T, int I, hipStream_t stream) {
-  PICO_REQUIRE(T >= 0 && I > 0, "pico_swiglu: bad sizes T=%d I=%d", T, I);
+template <int ACT>
+static int gated_act_launch(const void* gu, void* out, int dtype, int T, int I, float limit, float alpha, const char* who,
+                            hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && I > 0, "%s: bad sizes T=%d I=%d", who, T, I);
   if (T == 0) return 0;
   const size_t total = (size_t)T * I;
   if (dtype == PICO_DTYPE_BF16 && I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0) {
     const size_t total8 = total / 8;
-    swiglu_bf16x8_kernel<<<(unsigned)((total8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I / 8, total8);
+    gated_act_bf16x8_kernel<ACT><<<(unsigned)((total8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I / 8, total8, limit, alpha);
     PICO_LAUNCH_CHECK();
     return 0;
   }
   const unsigned blocks = (unsigned)((total + 255) / 256);
   if (dtype == PICO_DTYPE_F32)
-    swiglu_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total);
+    gated_act_kernel<float, ACT><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total, limit, alpha);
   else if (dtype == PICO_DTYPE_BF16)
-    swiglu_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total);
+    gated_act_kernel<bf16_t, ACT><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total, limit, alpha);
   else
-    PICO_REQUIRE(false, "pico_swiglu: unknown dtype %d", dtype);
+    PICO_REQUIRE(false, "%s: unknown dtype %d", who, dtype);
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int pico_swiglu(const void* gu, void* out, int dtype, int T, int I, hipStream_t stream) {
+  return gated_act_launch<ACT_SWIGLU>(gu, out, dtype, T, I, 0.f, 0.f, "pico_swiglu", stream);
+}
+
+extern "C" int pico_clipped_glu(const void* gu, void* out, int dtype, int T, int I, float limit, float alpha, hipStream_t stream) {
+  PICO_REQUIRE(limit > 0.f, "pico_clipped_glu: the limit must be positive");
+  return gated_act_launch<ACT_CLIPPED>(gu, out, dtype, T, I, limit, alpha, "pico_clipped_glu", stream);
+}
+
+// z[t][j] <- gelu_tanh(z[t][j]) * table[ids[t]][j], the table from its first column that is read (`ld` entries a row).
+template <typename T, typename TT>
+__global__ void gelu_token_kernel(T* __restrict__ z, const int* __restrict__ ids, const TT* __restrict__ table, long long ld,
+                                  int rows, int N, size_t total) {
+  const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const size_t t = idx / N, j = idx % N;
+  const size_t id = (size_t)min(max(ids[t], 0), rows - 1);
+  store_f32(z + idx, gelu_tanh_f(load_f32(z + idx)) * load_f32(table + id * ld + j));
+}
+
+extern "C" int pico_gelu_token(void* z, int dtype, const int* ids, const void* table, int table_dtype, long long ld, int rows,
+                               int T, int N, hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && N > 0 && ld >= N && rows > 0, "pico_gelu_token: bad sizes");
+  PICO_REQUIRE((dtype | 1) == 1 && (table_dtype | 1) == 1, "pico_gelu_token: unknown dtype");
+  if (T == 0) return 0;
+  const size_t total = (size_t)T * N;
+  const unsigned blocks = (unsigned)((total + 255) / 256);
+#define LAUNCH(TZ, TT) gelu_token_kernel<TZ, TT><<<blocks, 256, 0, stream>>>((TZ*)z, ids, (const TT*)table, ld, rows, N, total)
+  if (dtype == PICO_DTYPE_F32) {
+    if (table_dtype == PICO_DTYPE_F32) LAUNCH(float, float); else LAUNCH(float, bf16_t);
+  } else {
+    if (table_dtype == PICO_DTYPE_F32) LAUNCH(bf16_t, float); else LAUNCH(bf16_t, bf16_t);
+  }
+#undef LAUNCH
   PICO_LAUNCH_CHECK();
   return 0;
 }

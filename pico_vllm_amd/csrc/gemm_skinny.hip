@@ -53,7 +53,22 @@ struct TileRows {
 #define EPI_RELU2 3    // out bf16 [M, N] = max(x W^T + bias, 0)^2
 #define EPI_F32_ADD 4  // out float32 [M, N] += x W^T + bias (a residual stream; the k range is not split over the grid, so
                        // every element has one writer)
+#define EPI_CLIPPED 5  // W = [gate rows; up rows], out bf16 [M, N / 2] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up
+                       // clamped to -limit .. limit
+#define EPI_GELU_TOKEN 6   // out bf16 [M, N] = gelu_tanh(x W^T + bias) times columns of a table's row of the token
 #define MAX_SK_SLABS 8 // partial sums that a norm in front of a projection adds up
+
+// W's rows come in pairs (gate, up) whose sums meet in one output
+constexpr bool sk_paired(int epi) { return epi == EPI_SWIGLU || epi == EPI_CLIPPED; }
+
+// What some epilogues read beside the sums.
+struct SkExtra {
+  float limit, alpha;          // EPI_CLIPPED
+  const int* ids;              // EPI_GELU_TOKEN: the row of `table` (bf16, `ld` entries a row, clamped to `rows`) for every token
+  const bf16_t* table;         //   (already at the first column that is read)
+  long long ld;
+  int rows;
+};
 
 // The sums of one output tile when K is no multiple of 64 (any multiple of 8): operands go through
 // registers, lane (i, h) reads W[row i][k0 + 32 h ..] and the activations alike; k beyond the range
@@ -285,7 +300,7 @@ __device__ __forceinline__ float (*skinny_tile(const bf16_t* __restrict__ X, int
 template <int EPI>
 __device__ __forceinline__ TileRows skinny_rows(int tile, int rows, int N) {
   TileRows tr;
-  if (EPI == EPI_SWIGLU) {
+  if (sk_paired(EPI)) {
     const int I = N / 2;
     tr.row_a = min(tile * rows, I - 1);
     tr.row_b = I + tr.row_a;
@@ -304,7 +319,7 @@ __device__ __forceinline__ TileRows skinny_rows(int tile, int rows, int N) {
 template <int MT, int EPI>
 __device__ __forceinline__ void skinny_finish(float (*red)[MT][16][64], int tile, int rows, int a, int m0, int M, int N,
                                               const float* __restrict__ bias, void* __restrict__ out, int ldo,
-                                              long long slab_stride) {
+                                              long long slab_stride, const SkExtra& ex = SkExtra()) {
   const int lane = threadIdx.x & 63, col = lane & 31, h = lane >> 5;
   const int t0 = 8 * a + 4 * h;                      // this thread's first tile row
   if (t0 >= rows) return;
@@ -312,7 +327,7 @@ __device__ __forceinline__ void skinny_finish(float (*red)[MT][16][64], int tile
   for (int t = 0; t < MT; t++) {
     const int m = m0 + 32 * t + col;
     if (m >= M) continue;
-    if (EPI == EPI_SWIGLU) {
+    if (sk_paired(EPI)) {
       if (a >= 2) continue;
       const int I = N / 2, gi = tile * rows + t0;
       float v[4];
@@ -324,7 +339,13 @@ __device__ __forceinline__ void skinny_finish(float (*red)[MT][16][64], int tile
           g += red[w][t][4 * a + b][lane];
           u += red[w][t][4 * (a + 2) + b][lane];
         }
-        v[b] = g / (1.0f + __expf(-g)) * u;
+        if (EPI == EPI_CLIPPED) {
+          g = fminf(g, ex.limit);
+          u = fminf(fmaxf(u, -ex.limit), ex.limit);
+          v[b] = g / (1.0f + __expf(-ex.alpha * g)) * (u + 1.0f);
+        } else {
+          v[b] = g / (1.0f + __expf(-g)) * u;
+        }
       }
       bf16_t* o = (bf16_t*)out + (size_t)m * ldo + gi;
 #pragma unroll
@@ -343,6 +364,11 @@ __device__ __forceinline__ void skinny_finish(float (*red)[MT][16][64], int tile
           v[b] = fmaxf(v[b], 0.f);
           v[b] *= v[b];
         }
+      }
+      if (EPI == EPI_GELU_TOKEN) {
+        const bf16_t* e = ex.table + (size_t)min(max(ex.ids[m], 0), ex.rows - 1) * ex.ld;
+#pragma unroll
+        for (int b = 0; b < 4; b++) v[b] = gelu_tanh_f(v[b]) * bf16_to_f32(e[min(n + b, N - 1)]);
       }
       if (EPI == EPI_F32) {
         float* o = (float*)out + (size_t)blockIdx.y * slab_stride + (size_t)m * ldo + n;
@@ -370,7 +396,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_kernel(const bf16_t* __restri
                                                           const bf16_t* __restrict__ W, int ldw,
                                                           const float* __restrict__ bias, void* __restrict__ out,
                                                           int ldo, long long slab_stride, int M, int N, int K,
-                                                          int k_per_wg, int rows) {
+                                                          int k_per_wg, int rows, SkExtra ex) {
   __shared__ __attribute__((aligned(16))) char smem[sk_smem_bytes<MT, NX, FILL>()];
   const int wave = threadIdx.x >> 6;
   const int tile = blockIdx.x;
@@ -378,7 +404,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_kernel(const bf16_t* __restri
   const int k_begin = blockIdx.y * k_per_wg, k_end = min(K, k_begin + k_per_wg);
   float(*red)[MT][16][64] = skinny_tile<MT, TAIL, NX, FILL>(X, ldx, W, ldw, skinny_rows<EPI>(tile, rows, N), m0, M, k_begin, k_end, smem);
   constexpr int NWV = sk_waves<MT, NX, FILL>();
-  for (int a = wave; a < 4; a += NWV) skinny_finish<MT, EPI>(red, tile, rows, a, m0, M, N, bias, out, ldo, slab_stride);
+  for (int a = wave; a < 4; a += NWV) skinny_finish<MT, EPI>(red, tile, rows, a, m0, M, N, bias, out, ldo, slab_stride, ex);
 }
 
 // ---- one token: the norm in front of the projection inside the projection's launch -------------------
@@ -587,7 +613,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_pair_kernel(const bf16_t* __r
                                                                const bf16_t* __restrict__ W, int ldw,
                                                                const float* __restrict__ bias, void* __restrict__ out,
                                                                int ldo, long long slab_stride, int M, int N, int K,
-                                                               int k_per_wg, int rows) {
+                                                               int k_per_wg, int rows, SkExtra ex) {
   __shared__ __attribute__((aligned(16))) char smem[SK_PAIR_SMEM];
   const int wave = threadIdx.x >> 6;
   const int tile = 2 * blockIdx.x + (wave >> 1);     // of this wave while it streams
@@ -596,7 +622,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_pair_kernel(const bf16_t* __r
   skinny_stream_pair(X, ldx, W, ldw, skinny_rows<EPI>(tile, rows, N), m0, M, k_begin, k_end, smem);
   float(*red)[2][16][64] = reinterpret_cast<float(*)[2][16][64]>(smem);
   for (int item = wave; item < 8; item += 4)         // (tile of the pair, a)
-    skinny_finish<2, EPI>(red + 4 * (item >> 2), 2 * blockIdx.x + (item >> 2), rows, item & 3, m0, M, N, bias, out, ldo, slab_stride);
+    skinny_finish<2, EPI>(red + 4 * (item >> 2), 2 * blockIdx.x + (item >> 2), rows, item & 3, m0, M, N, bias, out, ldo, slab_stride, ex);
 }
 
 // How many rows of W (pairs of rows for the SwiGLU and rotation epilogues, `unit` = 2 rows) a tile gets:
@@ -654,18 +680,22 @@ extern "C" int pico_gemm_skinny_k_splits(int N, int K, int max_splits) {
 }
 
 // k_splits > 1 is allowed for EPI_F32 only: slab y (float32 [M, ldo]) lies at out + y * slab_stride and
-// holds the partial sum over its k range; the bias goes into slab 0.
+// holds the partial sum over its k range; the bias goes into slab 0.  limit, alpha: EPI_CLIPPED; ids [M], table [table_rows,
+// table_ld] (from its first column that is read): EPI_GELU_TOKEN.
 extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, const float* bias, void* out, int ldo,
-                                long long slab_stride, int epilogue, int M, int N, int K, int k_splits,
-                                hipStream_t stream) {
+                                long long slab_stride, int epilogue, int M, int N, int K, int k_splits, float limit, float alpha,
+                                const int* ids, const void* table, long long table_ld, int table_rows, hipStream_t stream) {
   PICO_REQUIRE(M > 0 && N > 0 && K > 0, "pico_gemm_skinny: bad sizes M=%d N=%d K=%d", M, N, K);
   PICO_REQUIRE(K % 8 == 0 && ldx % 8 == 0 && ldw % 8 == 0 && ldx >= K && ldw >= K,
                "pico_gemm_skinny: K and the row strides must be multiples of 8 (K=%d ldx=%d ldw=%d)", K, ldx, ldw);
   PICO_REQUIRE((uintptr_t)X % 16 == 0 && (uintptr_t)W % 16 == 0, "pico_gemm_skinny: operands must be 16-byte aligned");
-  PICO_REQUIRE(epilogue >= 0 && epilogue <= 4, "pico_gemm_skinny: unknown epilogue %d", epilogue);
+  PICO_REQUIRE(epilogue >= 0 && epilogue <= 6, "pico_gemm_skinny: unknown epilogue %d", epilogue);
   PICO_REQUIRE(k_splits >= 1 && (k_splits == 1 || epilogue == EPI_F32), "pico_gemm_skinny: only the float32 epilogue can split k over the grid");
-  PICO_REQUIRE(epilogue != EPI_SWIGLU || (N % 2 == 0 && bias == nullptr), "pico_gemm_skinny: SwiGLU needs an even N and no bias");
-  const int n_out = epilogue == EPI_SWIGLU ? N / 2 : N;
+  PICO_REQUIRE(!sk_paired(epilogue) || (N % 2 == 0 && bias == nullptr), "pico_gemm_skinny: gated activations need an even N and no bias");
+  PICO_REQUIRE(epilogue != EPI_CLIPPED || limit > 0.f, "pico_gemm_skinny: the clipped activation needs a positive limit");
+  PICO_REQUIRE(epilogue != EPI_GELU_TOKEN || (ids && table && table_ld >= N && table_rows > 0), "pico_gemm_skinny: the tokens' table is missing or too small");
+  const SkExtra ex{limit, alpha, ids, (const bf16_t*)table, table_ld, table_rows};
+  const int n_out = sk_paired(epilogue) ? N / 2 : N;
   PICO_REQUIRE(ldo >= n_out, "pico_gemm_skinny: output row stride too small");
   const int mt = M <= 32 ? 1 : 2;
   const int k_per_wg = ((K + k_splits - 1) / k_splits + 255) / 256 * 256;
@@ -674,8 +704,8 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   const bool tail = K % 64 != 0;
   // few rows and whole slices: the stream through LDS, with as many 8-token groups as hold tokens
   const int nx = tail ? 0 : (mt == 2 ? 8 : M <= 8 ? 1 : M <= 16 ? 2 : 4);
-  const int unit = epilogue == EPI_SWIGLU ? 2 : 1;
-  const int total = epilogue == EPI_SWIGLU ? N / 2 : N;
+  const int unit = sk_paired(epilogue) ? 2 : 1;
+  const int total = sk_paired(epilogue) ? N / 2 : N;
   // the tile height that fills the chip best; 33 to 64 tokens and whole slices: also whether two tiles of
   // W per workgroup, which share the activations, do better than one
   double cost1, cost2 = 0;
@@ -690,11 +720,13 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   if (pair) {
     dim3 pgrid((tiles + 1) / 2, ky, grid.z);
 #define LAUNCHP(EPI) \
-  gemm_skinny_pair_kernel<EPI><<<pgrid, 256, 0, stream>>>((const bf16_t*)X, ldx, (const bf16_t*)W, ldw, b0, out, ldo, slab_stride, M, N, K, k_per_wg, rows)
+  gemm_skinny_pair_kernel<EPI><<<pgrid, 256, 0, stream>>>((const bf16_t*)X, ldx, (const bf16_t*)W, ldw, b0, out, ldo, slab_stride, M, N, K, k_per_wg, rows, ex)
     if (epilogue == EPI_BF16) LAUNCHP(EPI_BF16);
     else if (epilogue == EPI_F32) LAUNCHP(EPI_F32);
     else if (epilogue == EPI_RELU2) LAUNCHP(EPI_RELU2);
     else if (epilogue == EPI_F32_ADD) LAUNCHP(EPI_F32_ADD);
+    else if (epilogue == EPI_CLIPPED) LAUNCHP(EPI_CLIPPED);
+    else if (epilogue == EPI_GELU_TOKEN) LAUNCHP(EPI_GELU_TOKEN);
     else LAUNCHP(EPI_SWIGLU);
 #undef LAUNCHP
     PICO_LAUNCH_CHECK();
@@ -709,7 +741,7 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   // tokens, two waves beyond), three or four of them a unit
   const bool many = workgroups > 2 * SK_COMPUTE_UNITS;
 #define LAUNCH4(MT, EPI, TAIL, NX, FILL) \
-  gemm_skinny_kernel<MT, EPI, TAIL, NX, FILL><<<grid, 64 * sk_waves<MT, NX, FILL>(), 0, stream>>>((const bf16_t*)X, ldx, (const bf16_t*)W, ldw, b0, out, ldo, slab_stride, M, N, K, k_per_wg, rows)
+  gemm_skinny_kernel<MT, EPI, TAIL, NX, FILL><<<grid, 64 * sk_waves<MT, NX, FILL>(), 0, stream>>>((const bf16_t*)X, ldx, (const bf16_t*)W, ldw, b0, out, ldo, slab_stride, M, N, K, k_per_wg, rows, ex)
 #define LAUNCH(EPI)                                               \
   do {                                                            \
     if (nx == 1 && many) LAUNCH4(1, EPI, false, 1, SK_MANY);      \
@@ -727,6 +759,8 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   else if (epilogue == EPI_F32) LAUNCH(EPI_F32);
   else if (epilogue == EPI_RELU2) LAUNCH(EPI_RELU2);
   else if (epilogue == EPI_F32_ADD) LAUNCH(EPI_F32_ADD);
+  else if (epilogue == EPI_CLIPPED) LAUNCH(EPI_CLIPPED);
+  else if (epilogue == EPI_GELU_TOKEN) LAUNCH(EPI_GELU_TOKEN);
   else LAUNCH(EPI_SWIGLU);
 #undef LAUNCH4
 #undef LAUNCH

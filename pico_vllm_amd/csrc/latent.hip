@@ -1,6 +1,7 @@
 // Attention through low-rank latents: what stands between the down projections and the attention kernel.
 //
-// A row of the first product holds [query latent (q_rank) | key/value latent (kv_rank) | rotated key part (rot)].
+// A row of the first product holds [query latent (q_rank) | key/value latent (kv_rank) | rotated key part (rot)]; q_rank 0:
+// the queries come from elsewhere (a full projection).
 //   cq = rmsnorm(query latent) * wq                      -> its own tensor, for the queries' up projection
 //   c  = rmsnorm(key/value latent) * wkv
 //   kr = the rotated key part turned by the token's angles (neighbouring pairs)
@@ -23,9 +24,11 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const T* __restrict
   const int t = blockIdx.x;
   const T* row = y + (size_t)t * ldy;
   float ss = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) { const float v = load_f32(row + i); ss = fmaf(v, v, ss); }
-  const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)q_rank + eps);
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) store_f32(cq + (size_t)t * q_rank + i, load_f32(row + i) * rq * wq[i]);
+  if (q_rank > 0) {
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) { const float v = load_f32(row + i); ss = fmaf(v, v, ss); }
+    const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) store_f32(cq + (size_t)t * q_rank + i, load_f32(row + i) * rq * wq[i]);
+  }
   const int slot = slots[t];
   if (slot < 0 || slot >= num_pages * P) return;        // a token that keeps nothing (padding of a recorded step)
   const T* lat = row + q_rank;
@@ -52,7 +55,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const T* __restrict
 extern "C" int pico_latent_prepare(const void* y, int ldy, int dtype, int q_rank, int kv_rank, int rot, const float* wq,
                                    const float* wkv, float eps, const float* cos_sin, const int* slots, void* cq,
                                    void* k_cache, void* v_cache, int T, int P, int num_pages, hipStream_t stream) {
-  PICO_REQUIRE(T >= 0 && q_rank > 0 && kv_rank > 0 && rot >= 0 && rot % 2 == 0 && ldy >= q_rank + kv_rank + rot && P > 0 && num_pages > 0,
+  PICO_REQUIRE(T >= 0 && q_rank >= 0 && (q_rank == 0 || (wq && cq)) && kv_rank > 0 && rot >= 0 && rot % 2 == 0 && ldy >= q_rank + kv_rank + rot && P > 0 && num_pages > 0,
                "pico_latent_prepare: bad sizes");
   PICO_REQUIRE(eps > 0.f, "pico_latent_prepare: eps must be positive");
   if (T == 0) return 0;

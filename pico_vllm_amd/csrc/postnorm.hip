@@ -3,6 +3,8 @@
 //   pico_norm_add:        x[t] += rms(y[t]) * w                          (y: the sublayer's output)
 //                         or, with two outputs a and b and a weight each,
 //                         x[t] += rms( (rms(a[t]) * wa + rms(b[t]) * wb) / 2 ) * w
+//   pico_norm_add_norm:   x[t] += rms(y[t]) * w, and out[t] = rms(x[t]) * w_next (the next sublayer's norm in front of it) or,
+//                         without w_next, x[t] itself in the activations' storage type
 //   pico_stream_rmsnorm:  x[t] <- rms(x[t]) * w
 //   rms(v) = v / sqrt(mean(v^2) + eps).  Both can leave a copy of the new x in the activations' storage type, which is
 //   what the next sublayer reads.
@@ -73,6 +75,86 @@ __global__ __launch_bounds__(1024) void norm_add_kernel(float* __restrict__ x, c
   }
 }
 
+// V neighbouring entries
+template <typename T, int V> __device__ __forceinline__ void load_v(const T* p, float* v) {
+  if constexpr (V == 1) {
+    v[0] = load_f32(p);
+  } else if constexpr (sizeof(T) == 4) {
+    const float4 r = *reinterpret_cast<const float4*>(p);
+    v[0] = r.x; v[1] = r.y; v[2] = r.z; v[3] = r.w;
+  } else {
+    const uint2 r = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(r.x << 16); v[1] = __uint_as_float(r.x & 0xffff0000u);
+    v[2] = __uint_as_float(r.y << 16); v[3] = __uint_as_float(r.y & 0xffff0000u);
+  }
+}
+template <typename T, int V> __device__ __forceinline__ void store_v(T* p, const float* v) {
+  if constexpr (V == 1) store_f32(p, v[0]);
+  else if constexpr (sizeof(T) == 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  else *reinterpret_cast<uint2*>(p) = make_uint2(pack2_bf16(v[0], v[1]), pack2_bf16(v[2], v[3]));
+}
+
+// Norm of the output, sum and norm of the sum with the row in registers: a thread owns VPT times V neighbouring entries,
+// thread i the entries (j * blockDim + i) * V ..; the number of threads goes with H alone, so a row's sums run in one order
+// whatever stands beside it.  All loads of a row are issued before the first sum.
+template <typename TY, typename TO, int V, int VPT>
+__global__ __launch_bounds__(1024) void norm_add_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, int slabs,
+                                                             size_t slab_stride, const float* __restrict__ w, float eps,
+                                                             const float* __restrict__ w_next, float eps_next, TO* __restrict__ out,
+                                                             int ld_out, int H) {
+  __shared__ float scratch[16];
+  const size_t base = (size_t)blockIdx.x * H;
+  float yv[VPT][V], xv[VPT][V], wv[VPT][V];
+  bool ok[VPT];
+#pragma unroll
+  for (int j = 0; j < VPT; j++) {
+    const int at = (j * (int)blockDim.x + (int)threadIdx.x) * V;
+    ok[j] = at < H;
+    const int i = ok[j] ? at : 0;
+    load_v<float, V>(x + base + i, xv[j]);
+    load_v<float, V>(w + i, wv[j]);
+    load_v<TY, V>(y + base + i, yv[j]);
+  }
+  for (int s = 1; s < slabs; s++) {
+    float more[VPT][V];
+#pragma unroll
+    for (int j = 0; j < VPT; j++) load_v<TY, V>(y + s * slab_stride + base + (ok[j] ? (j * (int)blockDim.x + (int)threadIdx.x) * V : 0), more[j]);
+#pragma unroll
+    for (int j = 0; j < VPT; j++)
+#pragma unroll
+      for (int k = 0; k < V; k++) yv[j][k] += more[j][k];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < VPT; j++)
+#pragma unroll
+    for (int k = 0; k < V; k++) ss = ok[j] ? fmaf(yv[j][k], yv[j][k], ss) : ss;
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
+  ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < VPT; j++) {
+#pragma unroll
+    for (int k = 0; k < V; k++) {
+      xv[j][k] += yv[j][k] * r * wv[j][k];
+      ss = ok[j] ? fmaf(xv[j][k], xv[j][k], ss) : ss;
+    }
+    if (ok[j]) store_v<float, V>(x + base + (j * (int)blockDim.x + (int)threadIdx.x) * V, xv[j]);
+  }
+  if (out == nullptr) return;
+  if (w_next) {
+#pragma unroll
+    for (int j = 0; j < VPT; j++) load_v<float, V>(w_next + (ok[j] ? (j * (int)blockDim.x + (int)threadIdx.x) * V : 0), wv[j]);
+    const float rn = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps_next);
+#pragma unroll
+    for (int j = 0; j < VPT; j++)
+#pragma unroll
+      for (int k = 0; k < V; k++) xv[j][k] *= rn * wv[j][k];
+  }
+#pragma unroll
+  for (int j = 0; j < VPT; j++)
+    if (ok[j]) store_v<TO, V>(out + (size_t)blockIdx.x * ld_out + (j * (int)blockDim.x + (int)threadIdx.x) * V, xv[j]);
+}
+
 template <typename TO>
 __global__ __launch_bounds__(256) void stream_rmsnorm_kernel(float* __restrict__ x, const float* __restrict__ w, float eps,
                                                              TO* __restrict__ copy, int H) {
@@ -132,6 +214,58 @@ extern "C" int pico_norm_add(float* x, const void* a, int a_dtype, int a_slabs, 
     default: LAUNCH(bf16_t, bf16_t, bf16_t); break;
   }
 #undef LAUNCH
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int pico_norm_add_norm(float* x, const void* y, int y_dtype, int slabs, long long slab_stride, const float* w, float eps,
+                                  const float* w_next, float eps_next, void* out, int out_dtype, int ld_out, int T, int H,
+                                  hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && H > 0 && H <= POSTNORM_MAX_H, "pico_norm_add_norm: a width of 1 to %d, got %d", POSTNORM_MAX_H, H);
+  PICO_REQUIRE(x && y && w && slabs >= 1 && (slabs == 1 || y_dtype == PICO_DTYPE_F32), "pico_norm_add_norm: bad operands (partial sums are float32)");
+  PICO_REQUIRE(eps > 0.f && (w_next == nullptr || (eps_next > 0.f && out)) && (out == nullptr || ld_out >= H), "pico_norm_add_norm: bad operands");
+  PICO_REQUIRE((y_dtype | 1) == 1 && (out_dtype | 1) == 1, "pico_norm_add_norm: unknown dtype");
+  if (T == 0) return 0;
+  const uintptr_t all = (uintptr_t)x | (uintptr_t)y | (uintptr_t)w | (uintptr_t)w_next | (uintptr_t)out;
+  // (every pointer on 16 bytes and rows of whole fours: then so is every row, or on 8 bytes where storage is bfloat16)
+  const bool four = H % 4 == 0 && all % 16 == 0 && (out == nullptr || ld_out % 4 == 0) && (slabs == 1 || slab_stride % 4 == 0);
+  const int units = four ? H / 4 : H;
+  const int vpt = units <= 1024 ? 1 : units <= 4096 ? 4 : 16;
+  const int threads = ((units + vpt - 1) / vpt + 63) / 64 * 64;
+#define LAUNCH(TY, TO, V, VPT)                                                                                                   \
+  norm_add_norm_kernel<TY, TO, V, VPT><<<T, threads, 0, stream>>>(x, (const TY*)y, slabs, (size_t)slab_stride, w, eps, w_next,   \
+                                                                  eps_next, (TO*)out, ld_out, H)
+#define PICK(TY, TO)                              \
+  do {                                            \
+    if (four && vpt == 1) LAUNCH(TY, TO, 4, 1);   \
+    else if (four) LAUNCH(TY, TO, 4, 4);          \
+    else if (vpt == 1) LAUNCH(TY, TO, 1, 1);      \
+    else if (vpt == 4) LAUNCH(TY, TO, 1, 4);      \
+    else LAUNCH(TY, TO, 1, 16);                   \
+  } while (0)
+  if (y_dtype == PICO_DTYPE_F32) {
+    if (out_dtype == PICO_DTYPE_F32) PICK(float, float); else PICK(float, bf16_t);
+  } else {
+    if (out_dtype == PICO_DTYPE_F32) PICK(bf16_t, float); else PICK(bf16_t, bf16_t);
+  }
+#undef PICK
+#undef LAUNCH
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+// out[t][i] = x[t][i] in the storage type `dtype`; rows of the output lie ld_out apart.
+template <typename T>
+__global__ __launch_bounds__(256) void store_rows_kernel(const float* __restrict__ x, T* __restrict__ out, int ld_out, int H) {
+  for (int i = threadIdx.x; i < H; i += blockDim.x) store_f32(out + (size_t)blockIdx.x * ld_out + i, x[(size_t)blockIdx.x * H + i]);
+}
+
+extern "C" int pico_store_rows(const float* x, void* out, int dtype, int ld_out, int T, int H, hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && H > 0 && ld_out >= H, "pico_store_rows: bad sizes");
+  if (T == 0) return 0;
+  if (dtype == PICO_DTYPE_F32) store_rows_kernel<float><<<T, 256, 0, stream>>>(x, (float*)out, ld_out, H);
+  else if (dtype == PICO_DTYPE_BF16) store_rows_kernel<bf16_t><<<T, 256, 0, stream>>>(x, (bf16_t*)out, ld_out, H);
+  else PICO_REQUIRE(false, "pico_store_rows: unknown dtype %d", dtype);
   PICO_LAUNCH_CHECK();
   return 0;
 }

@@ -1,8 +1,9 @@
 // A selective state-space mixer: a short causal convolution per channel and a recurrence whose decay, input and
 // output weights depend on the token.
 //
-//   xc[t][c] = silu(bias[c] + sum_j w[j][c] * x[t - (taps - 1) + j][c])          zeros before a sequence's start; w is kept
-//                                                                            tap by tap, [taps, C]: neighbours read neighbours
+//   xc[t][c] = act(bias[c] + sum_j w[j][c] * x[t - (taps - 1) + j][c])          zeros before a sequence's start; act is
+//                                                                           silu, or nothing; w is kept tap by tap,
+//                                                                           [taps, C]: neighbours read neighbours
 //   dt[t][c] = softplus(dtp[t][c] + dt_bias[c]),   A[c][n] = -exp(A_log[c][n])
 //   S[c][n] <- exp(dt A) S + dt xc[t][c] B[t][n];   y[t][c] = sum_n S[c][n] C[t][n] + D[c] xc[t][c]
 //   out[t][c] = y[t][c] * silu(z[t][c])
@@ -15,6 +16,8 @@
 #define SSM_MAX_TAPS 16
 
 __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
+// what follows the convolution: silu, or nothing
+__device__ __forceinline__ float conv_act(float v, int silu) { return silu ? silu_f(v) : v; }
 // the decay exp(dt A) of an element: the library's exponential in the 32-bit engine; with bfloat16 storage the
 // hardware's (exp2 of the argument times log2 e; the argument is at most 0, the relative error a few 1e-7)
 template <typename T> __device__ __forceinline__ float decay_exp(float v);
@@ -27,7 +30,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
                                                           const float* __restrict__ bias, const int* __restrict__ token_seq,
                                                           const int* __restrict__ cu_seqlens,
                                                           const int* __restrict__ state_slots, const float* __restrict__ state,
-                                                          int num_slots, int C, int N, int taps, T* __restrict__ out) {
+                                                          int num_slots, int C, int N, int taps, int silu, T* __restrict__ out) {
   const int t = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int b = token_seq[t], first = cu_seqlens[b];
@@ -39,7 +42,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
     const float v = src >= first ? load_f32(x + (size_t)src * ldx + c) : hist[(taps - 1) + (src - first)];
     acc = fmaf(w[(size_t)j * C + c], v, acc);
   }
-  store_f32(out + (size_t)t * C + c, silu_f(acc));
+  store_f32(out + (size_t)t * C + c, conv_act(acc, silu));
 }
 
 // The same for bfloat16 with eight neighbouring channels a thread (16-byte accesses; C and the row stride multiples of 8).
@@ -48,7 +51,7 @@ __global__ __launch_bounds__(256) void causal_conv8_kernel(const bf16_t* __restr
                                                            const float* __restrict__ bias, const int* __restrict__ token_seq,
                                                            const int* __restrict__ cu_seqlens,
                                                            const int* __restrict__ state_slots, const float* __restrict__ state,
-                                                           int num_slots, int C, int N, int taps, bf16_t* __restrict__ out) {
+                                                           int num_slots, int C, int N, int taps, int silu, bf16_t* __restrict__ out) {
   const int t = blockIdx.x, c0 = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
   if (c0 >= C) return;
   const int b = token_seq[t], first = cu_seqlens[b];
@@ -74,10 +77,10 @@ __global__ __launch_bounds__(256) void causal_conv8_kernel(const bf16_t* __restr
     acc[4] = fmaf(w1.x, v[4], acc[4]); acc[5] = fmaf(w1.y, v[5], acc[5]); acc[6] = fmaf(w1.z, v[6], acc[6]); acc[7] = fmaf(w1.w, v[7], acc[7]);
   }
   uint4 o;
-  o.x = pack2_bf16(silu_f(acc[0]), silu_f(acc[1]));
-  o.y = pack2_bf16(silu_f(acc[2]), silu_f(acc[3]));
-  o.z = pack2_bf16(silu_f(acc[4]), silu_f(acc[5]));
-  o.w = pack2_bf16(silu_f(acc[6]), silu_f(acc[7]));
+  o.x = pack2_bf16(conv_act(acc[0], silu), conv_act(acc[1], silu));
+  o.y = pack2_bf16(conv_act(acc[2], silu), conv_act(acc[3], silu));
+  o.z = pack2_bf16(conv_act(acc[4], silu), conv_act(acc[5], silu));
+  o.w = pack2_bf16(conv_act(acc[6], silu), conv_act(acc[7], silu));
   *reinterpret_cast<uint4*>(out + (size_t)t * C + c0) = o;
 }
 
@@ -105,7 +108,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void causal_conv_step_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ w,
                                                                const float* __restrict__ bias, const int* __restrict__ cu_seqlens,
                                                                const int* __restrict__ state_slots, float* __restrict__ state,
-                                                               int num_slots, int C, int N, int taps, T* __restrict__ out) {
+                                                               int num_slots, int C, int N, int taps, int silu, T* __restrict__ out) {
   const int b = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int t = cu_seqlens[b], slot = state_slots[b];
@@ -121,12 +124,12 @@ __global__ __launch_bounds__(256) void causal_conv_step_kernel(const T* __restri
   acc = fmaf(w[(size_t)(taps - 1) * C + c], xv, acc);
   for (int j = 0; j + 1 < taps - 1; j++) hist[j] = keep[j + 1];
   if (taps > 1) hist[taps - 2] = xv;
-  store_f32(out + (size_t)t * C + c, silu_f(acc));
+  store_f32(out + (size_t)t * C + c, conv_act(acc, silu));
 }
 
 extern "C" int pico_causal_conv(const void* x, int ldx, int dtype, const float* w, const float* bias, const int* token_seq,
                                 const int* cu_seqlens, const int* state_slots, float* state, int num_slots, int T, int B,
-                                int C, int N, int taps, void* out, int single, hipStream_t stream) {
+                                int C, int N, int taps, void* out, int single, int silu, hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && B >= 0 && C > 0 && N >= 0 && taps >= 1 && taps <= SSM_MAX_TAPS && ldx >= C && num_slots > 0,
                "pico_causal_conv: bad sizes (1 to %d taps)", SSM_MAX_TAPS);
   if (T == 0 || B == 0) return 0;
@@ -136,10 +139,10 @@ extern "C" int pico_causal_conv(const void* x, int ldx, int dtype, const float* 
     PICO_REQUIRE(T == B, "pico_causal_conv: a step of single tokens has as many tokens as sequences");
     if (dtype == PICO_DTYPE_F32)
       causal_conv_step_kernel<float><<<dim3(B, cb), 256, 0, stream>>>((const float*)x, ldx, w, bias, cu_seqlens, state_slots, state,
-                                                                      num_slots, C, N, taps, (float*)out);
+                                                                      num_slots, C, N, taps, silu, (float*)out);
     else if (dtype == PICO_DTYPE_BF16)
       causal_conv_step_kernel<bf16_t><<<dim3(B, cb), 256, 0, stream>>>((const bf16_t*)x, ldx, w, bias, cu_seqlens, state_slots, state,
-                                                                       num_slots, C, N, taps, (bf16_t*)out);
+                                                                       num_slots, C, N, taps, silu, (bf16_t*)out);
     else
       PICO_REQUIRE(false, "pico_causal_conv: unknown dtype %d", dtype);
     PICO_LAUNCH_CHECK();
@@ -147,16 +150,16 @@ extern "C" int pico_causal_conv(const void* x, int ldx, int dtype, const float* 
   }
   if (dtype == PICO_DTYPE_F32) {
     causal_conv_kernel<float><<<dim3(T, cb), 256, 0, stream>>>((const float*)x, ldx, w, bias, token_seq, cu_seqlens, state_slots,
-                                                               state, num_slots, C, N, taps, (float*)out);
+                                                               state, num_slots, C, N, taps, silu, (float*)out);
     if (taps > 1)
       conv_history_kernel<float><<<dim3(B, cb), 256, 0, stream>>>((const float*)x, ldx, cu_seqlens, state_slots, state, num_slots, C, N, taps);
   } else if (dtype == PICO_DTYPE_BF16) {
     if (C % 8 == 0 && ldx % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)w % 16 == 0)
       causal_conv8_kernel<<<dim3(T, (C / 8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)x, ldx, w, bias, token_seq, cu_seqlens,
-                                                                            state_slots, state, num_slots, C, N, taps, (bf16_t*)out);
+                                                                            state_slots, state, num_slots, C, N, taps, silu, (bf16_t*)out);
     else
       causal_conv_kernel<bf16_t><<<dim3(T, cb), 256, 0, stream>>>((const bf16_t*)x, ldx, w, bias, token_seq, cu_seqlens, state_slots,
-                                                                  state, num_slots, C, N, taps, (bf16_t*)out);
+                                                                  state, num_slots, C, N, taps, silu, (bf16_t*)out);
     if (taps > 1)
       conv_history_kernel<bf16_t><<<dim3(B, cb), 256, 0, stream>>>((const bf16_t*)x, ldx, cu_seqlens, state_slots, state, num_slots, C, N, taps);
   } else {

@@ -196,6 +196,19 @@ def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.T
     return out
 
 
+def clipped_glu(gate_up: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
+    """[gate | up] [T, 2 I] -> [T, I]: g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = up clamped to
+    -limit .. limit."""
+    _gpu(gate_up)
+    T, I2 = gate_up.shape
+    if I2 % 2 or not gate_up.is_contiguous() or not limit > 0:
+        raise KernelError("clipped_glu: input must be contiguous [T, 2 I] and the limit positive")
+    out = torch.empty(T, I2 // 2, dtype=gate_up.dtype, device=gate_up.device)
+    lib = library.core()
+    _check(lib, lib.pico_clipped_glu(_ptr(gate_up), _ptr(out), _dt(gate_up), T, I2 // 2, c_float(limit), c_float(alpha), _stream()))
+    return out
+
+
 def gemm_f32(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
              out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """float32 out = a @ w.T + bias with plain FMA.  a: [M, K] float32 or bfloat16 (rows may be
@@ -243,7 +256,7 @@ def gemm_bf16(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = N
     return out
 
 
-EPI_BF16, EPI_F32, EPI_SWIGLU, EPI_RELU2, EPI_F32_ADD = 0, 1, 2, 3, 4
+EPI_BF16, EPI_F32, EPI_SWIGLU, EPI_RELU2, EPI_F32_ADD, EPI_CLIPPED, EPI_GELU_TOKEN = 0, 1, 2, 3, 4, 5, 6
 MAX_HEAD_DIM = 256          # the largest head size any attention kernel takes
 
 
@@ -271,11 +284,14 @@ def skinny_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
 
 
 def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None, epilogue: int = EPI_BF16,
-                k_splits: int = 1, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                k_splits: int = 1, out: Optional[torch.Tensor] = None, clip: Optional[tuple] = None,
+                token_rows: Optional[tuple] = None) -> torch.Tensor:
     """a [M <= 64, K] x w [N, K]^T, both bfloat16.  EPI_BF16 -> bf16 [M, N]; EPI_F32 -> float32 [M, N], or with
     k_splits > 1 a stack [k_splits, M, N] of partial sums (bias in the first); EPI_SWIGLU (w = [gate; up])
     -> bf16 [M, N / 2] = silu(gate) * up; EPI_RELU2 -> bf16 [M, N] = max(x w^T + bias, 0)^2; EPI_F32_ADD: ``out``
-    (contiguous float32 [M, N], a residual stream) += x w^T + bias, every element by one writer."""
+    (contiguous float32 [M, N], a residual stream) += x w^T + bias, every element by one writer; EPI_CLIPPED (w = [gate;
+    up], ``clip`` = (limit, alpha)) -> bf16 [M, N / 2] as ``clipped_glu``; EPI_GELU_TOKEN (``token_rows`` = (ids int32 [M],
+    table bf16 [rows, columns], first column)) -> bf16 [M, N] as ``gelu_token``."""
     _gpu(a, w, bias)
     M, K = a.shape
     N, K2 = w.shape
@@ -297,18 +313,48 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
         shape = (M, N) if k_splits == 1 else (k_splits, M, N)
         out = torch.empty(shape, dtype=torch.float32, device=a.device)
         ldo = N
-    elif epilogue == EPI_SWIGLU:
+    elif epilogue in (EPI_SWIGLU, EPI_CLIPPED):
         if N % 2:
-            raise KernelError("gemm_skinny: SwiGLU needs an even number of weight rows")
+            raise KernelError("gemm_skinny: gated activations need an even number of weight rows")
         out = torch.empty(M, N // 2, dtype=torch.bfloat16, device=a.device)
         ldo = N // 2
     else:
         out = torch.empty(M, N, dtype=torch.bfloat16, device=a.device)
         ldo = N
+    limit, alpha = clip if clip is not None else (0.0, 0.0)
+    ids = table = None
+    rows = ld = 0
+    if epilogue == EPI_GELU_TOKEN:
+        ids, table, col = token_rows
+        rows, ld = _check_token_rows(ids, table, col, M, N)
+        if table.dtype != torch.bfloat16:
+            raise KernelError("gemm_skinny: the tokens' table must be bfloat16")
+        table = table[:, col:]
     lib = library.core()
     _check(lib, lib.pico_gemm_skinny(_ptr(a), a.stride(0) if M > 1 else K, _ptr(w), w.stride(0), _ptr(bias), _ptr(out),
-                                     ldo, c_ll(M * N), epilogue, M, N, K, k_splits, _stream()))
+                                     ldo, c_ll(M * N), epilogue, M, N, K, k_splits, c_float(limit), c_float(alpha), _ptr(ids),
+                                     _ptr(table), c_ll(ld), rows, _stream()))
     return out
+
+
+def _check_token_rows(ids, table, col, T, N):
+    _gpu(ids, table)
+    _i32(ids, "token ids", T)
+    if table.dim() != 2 or table.stride(1) != 1 or col < 0 or col + N > table.shape[1]:
+        raise KernelError(f"the tokens' table must be [rows, >= {col + N}] with unit stride along the row")
+    return table.shape[0], table.stride(0)
+
+
+def gelu_token(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, col: int) -> torch.Tensor:
+    """z (contiguous [T, N], in place) <- gelu_tanh(z) * table[ids, col : col + N] in float32; returns z."""
+    _gpu(z)
+    T, N = z.shape
+    if not z.is_contiguous():
+        raise KernelError("gelu_token: z must be contiguous")
+    rows, ld = _check_token_rows(ids, table, col, T, N)
+    lib = library.core()
+    _check(lib, lib.pico_gelu_token(_ptr(z), _dt(z), _ptr(ids), _ptr(table[:, col:]), _dt(table), c_ll(ld), rows, T, N, _stream()))
+    return z
 
 
 @functools.lru_cache(maxsize=None)
@@ -1049,9 +1095,9 @@ def pair_embed(resid: torch.Tensor, table: torch.Tensor, ctx, last: torch.Tensor
 
 
 # ---- attention through latents ---------------------------------------------------------------------------------------
-def latent_prepare(y: torch.Tensor, q_rank: int, kv_rank: int, rot: int, wq: torch.Tensor, wkv: torch.Tensor, eps: float,
-                   cos_sin: Optional[torch.Tensor], slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
-    """y [T, q_rank + kv_rank + rot]: returns the normed query latent [T, q_rank]; writes the normed key/value latent and
+def latent_prepare(y: torch.Tensor, q_rank: int, kv_rank: int, rot: int, wq: Optional[torch.Tensor], wkv: torch.Tensor, eps: float,
+                   cos_sin: Optional[torch.Tensor], slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor) -> Optional[torch.Tensor]:
+    """y [T, q_rank + kv_rank + rot]: returns the normed query latent [T, q_rank] (q_rank 0: None); writes the normed key/value latent and
     the turned rotated key part into the cache (K rows [latent | rotated part], V columns the latent again)."""
     _gpu(y, wq, wkv, cos_sin, slots, k_cache, v_cache)
     T = y.shape[0]
@@ -1060,11 +1106,13 @@ def latent_prepare(y: torch.Tensor, q_rank: int, kv_rank: int, rot: int, wq: tor
     pages, P = _check_cache2(k_cache, v_cache, 1, kv_rank + rot, kv_rank)
     if k_cache.dtype != y.dtype:
         raise KernelError("cache and activations differ in dtype")
+    if q_rank and wq is None:
+        raise KernelError("latent_prepare: a query latent comes with its norm's weight")
     _vec(wq, q_rank, "the query latent's norm weight"); _vec(wkv, kv_rank, "the key/value latent's norm weight")
     _i32(slots, "slots", T)
     if rot:
         _check_table(cos_sin, T, rot // 2)
-    cq = torch.empty(T, q_rank, dtype=y.dtype, device=y.device)
+    cq = torch.empty(T, q_rank, dtype=y.dtype, device=y.device) if q_rank else None
     lib = library.core()
     _check(lib, lib.pico_latent_prepare(_ptr(y), y.stride(0) if T > 1 else y.shape[1], _dt(y), q_rank, kv_rank, rot, _ptr(wq),
                                         _ptr(wkv), c_float(eps), _ptr(cos_sin), _ptr(slots), _ptr(cq), _ptr(k_cache),
@@ -1119,9 +1167,9 @@ SSM_MAX_TAPS, SSM_MAX_STATE = 16, 256
 
 
 def causal_conv(x: torch.Tensor, channels: int, w: torch.Tensor, bias: torch.Tensor, ctx, state: torch.Tensor, n_state: int,
-                single: bool = False) -> torch.Tensor:
-    """silu(bias + the causal convolution of the first ``channels`` columns of x with w [taps, channels] (tap by tap,
-    the last row the current token's)) for every
+                single: bool = False, activation: str = "silu") -> torch.Tensor:
+    """act(bias + the causal convolution of the first ``channels`` columns of x with w [taps, channels] (tap by tap,
+    the last row the current token's)), act being silu or ("none") nothing, for every
     sequence of the step; inputs before a portion come from the slot's history (``state`` float32
     [slots, channels, n_state + taps - 1], its last taps - 1 columns), which is brought up to date.  ``single``: every
     sequence of the step brings one token (one launch makes the convolution and the history)."""
@@ -1135,13 +1183,16 @@ def causal_conv(x: torch.Tensor, channels: int, w: torch.Tensor, bias: torch.Ten
     _vec(bias, channels, "the convolution's bias")          # None: no bias
     if state.dtype != torch.float32 or state.dim() != 3 or tuple(state.shape[1:]) != (channels, n_state + taps - 1) or not state.is_contiguous():
         raise KernelError(f"causal_conv: the state must be contiguous float32 [slots, {channels}, {n_state + taps - 1}]")
+    if activation not in ("silu", "none"):
+        raise KernelError(f"causal_conv: activation {activation!r} is not known (silu, none)")
     B = ctx.num_seqs
     _i32(ctx.token_seq, "token_seq", T); _i32(ctx.cu_seqlens, "cu_seqlens", B + 1); _i32(ctx.state_slots, "state_slots", B)
     out = torch.empty(T, channels, dtype=x.dtype, device=x.device)
     lib = library.core()
     _check(lib, lib.pico_causal_conv(_ptr(x), x.stride(0) if T > 1 else x.shape[1], _dt(x), _ptr(w), _ptr(bias), _ptr(ctx.token_seq),
                                      _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), _ptr(state), state.shape[0], T, B, channels,
-                                     n_state, taps, _ptr(out), 1 if single and T == B else 0, _stream()))
+                                     n_state, taps, _ptr(out), 1 if single and T == B else 0, 1 if activation == "silu" else 0,
+                                     _stream()))
     return out
 
 
@@ -1246,6 +1297,42 @@ def norm_add(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: fl
                                   _ptr(weight2), c_ll(T * H), _ptr(weight), c_float(eps), _ptr(copy),
                                   _DT[copy_dtype] if copy_dtype is not None else F32, T, H, _stream()))
     return copy
+
+
+def norm_add_norm(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,
+                  next_eps: float = 0.0, out: Optional[torch.Tensor] = None,
+                  out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """resid (float32 [T, H], in place) += rms(y) * weight; y: [T, H], or a float32 stack [S, T, H] whose slabs are added up
+    first.  The same launch leaves rows beside the stream, in ``out`` ([T, H], row stride free) or a tensor made here of
+    ``out_dtype``: the new stream itself or, with ``next_weight``, its RMS norm with that weight.  Neither given: nothing."""
+    _gpu(resid, y, weight, next_weight, out)
+    T, H = resid.shape
+    if resid.dtype != torch.float32 or not resid.is_contiguous():
+        raise KernelError("the residual stream must be contiguous float32")
+    _vec(weight, H, "norm weight"); _vec(next_weight, H, "the next norm's weight")
+    slabs = _delta_like(resid, y, "norm_add_norm")
+    if out is None and out_dtype is not None:
+        out = torch.empty(T, H, dtype=out_dtype, device=resid.device)
+    if out is not None and (tuple(out.shape) != (T, H) or out.stride(1) != 1):
+        raise KernelError("norm_add_norm: the rows left beside the stream are [T, H] with unit stride along the row")
+    if next_weight is not None and out is None:
+        raise KernelError("norm_add_norm: the next norm's rows need a place")
+    lib = library.core()
+    _check(lib, lib.pico_norm_add_norm(_ptr(resid), _ptr(y), _dt(y), slabs, c_ll(T * H), _ptr(weight), c_float(eps), _ptr(next_weight),
+                                       c_float(next_eps), _ptr(out), _dt(out) if out is not None else F32,
+                                       out.stride(0) if out is not None and T > 1 else H, T, H, _stream()))
+    return out
+
+
+def store_rows(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out ([T, H], row stride free, float32 or bfloat16) <- x (contiguous float32 [T, H])."""
+    _gpu(x, out)
+    T, H = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous() or tuple(out.shape) != (T, H) or out.stride(1) != 1:
+        raise KernelError("store_rows: contiguous float32 rows and an equally shaped output with unit stride along the row")
+    lib = library.core()
+    _check(lib, lib.pico_store_rows(_ptr(x), _ptr(out), _dt(out), out.stride(0) if T > 1 else H, T, H, _stream()))
+    return out
 
 
 def stream_rmsnorm(resid: torch.Tensor, weight: torch.Tensor, eps: float, copy_dtype: Optional[torch.dtype] = None):
@@ -1452,4 +1539,84 @@ def gated_group_norm(y: torch.Tensor, x: torch.Tensor, z: torch.Tensor, d: torch
     _check(lib, lib.pico_gated_group_norm(_ptr(y), _ptr(x), x.stride(0) if T > 1 else x.shape[1], _ptr(z),
                                           z.stride(0) if T > 1 else z.shape[1], _dt(x), _ptr(d), _ptr(weight), c_float(eps), _ptr(out),
                                           T, heads, dv, groups, _stream()))
+    return out
+
+
+# ---- the gated linear recurrence with one state element a channel -----------------------------------------------------------
+LRU_MAX_TAPS, LRU_MAX_PART, LRU_CHUNK = 16, 8192, 64
+
+
+def _check_lru(rows, y, w, b_r, b_i, decay, ctx, state, hist, who):
+    """(T, sequences, channels, parts) of a recurrence's operands: rows [T, >= C], y [T, >= C] (row strides free), w = (ra,
+    ri) [parts, n, n] each of the activations' dtype, vectors float32 [C], state float32 [slots, C, 1 + hist]."""
+    wr, wi = w
+    _gpu(rows, y, wr, wi, b_r, b_i, decay, state)
+    T = rows.shape[0]
+    parts, n = wr.shape[0], wr.shape[1]
+    C = parts * n
+    if not 1 <= n <= LRU_MAX_PART or not 0 <= hist < LRU_MAX_TAPS:
+        raise KernelError(f"{who}: parts of at most {LRU_MAX_PART} channels and at most {LRU_MAX_TAPS} taps")
+    for t in (wr, wi):
+        if t.dim() != 3 or tuple(t.shape) != (parts, n, n) or not t.is_contiguous() or t.dtype != rows.dtype:
+            raise KernelError(f"{who}: the gates' matrices must be contiguous [parts, n, n] of the activations' dtype")
+    for t in (rows, y):
+        if t.dim() != 2 or t.shape[0] != T or t.stride(1) != 1 or t.shape[1] < C or t.dtype != rows.dtype:
+            raise KernelError(f"{who}: the rows do not hold the channels")
+    _vec(b_r, C, "a gate's bias"); _vec(b_i, C, "a gate's bias"); _vec(decay, C, "the decays")
+    if state.dtype != torch.float32 or state.dim() != 3 or tuple(state.shape[1:]) != (C, 1 + hist) or not state.is_contiguous():
+        raise KernelError(f"{who}: the state must be contiguous float32 [slots, {C}, {1 + hist}]")
+    B = ctx.num_seqs
+    _i32(ctx.token_seq, "token_seq", T); _i32(ctx.cu_seqlens, "cu_seqlens", B + 1); _i32(ctx.state_slots, "state_slots", B)
+    return T, B, C, parts
+
+
+def lru_scan(u: torch.Tensor, y: torch.Tensor, w: tuple, b_r: torch.Tensor, b_i: torch.Tensor, decay: torch.Tensor, ctx,
+             state: torch.Tensor, hist: int, w_out_in: Optional[tuple] = None, chunked: bool = False) -> torch.Tensor:
+    """r = sigmoid(ra u + b_r), i = sigmoid(ri u + b_i) part by part, a = exp(decay r), S <- a S + sqrt(1 - a^2) i u channel by
+    channel from every sequence's state slot (``state`` float32 [slots, C, 1 + hist], entry 0; updated in place); returns
+    S * gelu_tanh(y) [T, C] in u's dtype.  u contiguous [T, C]; y [T, >= C] (row stride free); w = (ra, ri) laid out [parts,
+    inner, output].  ``chunked`` (bfloat16, parts of a multiple of 8 channels; w_out_in: the matrices [parts, output,
+    inner]): chunks of LRU_CHUNK tokens side by side, the gates on the matrix cores: the same sums in another order."""
+    T, B, C, parts = _check_lru(u, y, w_out_in if chunked else w, b_r, b_i, decay, ctx, state, hist, "lru_scan")
+    if not u.is_contiguous() or u.shape[1] != C:
+        raise KernelError(f"lru_scan: u must be contiguous [T, {C}]")
+    dev = u.device
+    out = torch.empty(T, C, dtype=u.dtype, device=dev)
+    one = torch.empty(T, C, dtype=torch.float32, device=dev)
+    two = torch.empty(T, C, dtype=torch.float32, device=dev)
+    lib = library.core()
+    ldy = y.stride(0) if T > 1 else y.shape[1]
+    if not chunked:
+        _check(lib, lib.pico_lru_scan(_ptr(u), _ptr(y), ldy, _dt(u), _ptr(w[0]), _ptr(w[1]), _ptr(b_r), _ptr(b_i), _ptr(decay),
+                                      _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), _ptr(state), state.shape[0], T, B, C, parts, hist,
+                                      _ptr(one), _ptr(two), _ptr(out), _stream()))
+        return out
+    max_chunks = max(1, -(-T // LRU_CHUNK))
+    ws_s = torch.empty(B * max_chunks, C, dtype=torch.float32, device=dev)
+    ws_l = torch.empty(B * max_chunks, C, dtype=torch.float32, device=dev)
+    _check(lib, lib.pico_lru_chunks(_ptr(u), _ptr(y), ldy, _dt(u), _ptr(w_out_in[0]), _ptr(w_out_in[1]), _ptr(b_r), _ptr(b_i),
+                                    _ptr(decay), _ptr(ctx.token_seq), _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), _ptr(state),
+                                    state.shape[0], T, B, C, parts, hist, max_chunks, _ptr(one), _ptr(two), _ptr(ws_s), _ptr(ws_l),
+                                    _ptr(out), _stream()))
+    return out
+
+
+def lru_step(x: torch.Tensor, y: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, w: tuple, b_r: torch.Tensor,
+             b_i: torch.Tensor, decay: torch.Tensor, ctx, state: torch.Tensor) -> torch.Tensor:
+    """A step of single tokens in one launch: u = bias + causal convolution of x (``causal_conv`` without activation), then
+    as ``lru_scan``.  x, y [T, >= C] (row strides free); conv_w float32 [taps, C]; state [slots, C, taps]."""
+    hist = conv_w.shape[0] - 1
+    T, B, C, parts = _check_lru(x, y, w, b_r, b_i, decay, ctx, state, hist, "lru_step")
+    _gpu(conv_w, conv_b)
+    if T != B:
+        raise KernelError("lru_step: every sequence of the step brings one token")
+    if conv_w.dtype != torch.float32 or tuple(conv_w.shape) != (hist + 1, C) or not conv_w.is_contiguous() or conv_b is None:
+        raise KernelError(f"lru_step: the taps are contiguous float32 [taps, {C}] and come with a bias")
+    _vec(conv_b, C, "the convolution's bias")
+    out = torch.empty(T, C, dtype=x.dtype, device=x.device)
+    lib = library.core()
+    _check(lib, lib.pico_lru_step(_ptr(x), x.stride(0) if T > 1 else x.shape[1], _ptr(y), y.stride(0) if T > 1 else y.shape[1], _dt(x),
+                                  _ptr(conv_w), _ptr(conv_b), _ptr(w[0]), _ptr(w[1]), _ptr(b_r), _ptr(b_i), _ptr(decay),
+                                  _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), _ptr(state), state.shape[0], T, B, C, parts, hist,
+                                  _ptr(out), _stream()))
     return out

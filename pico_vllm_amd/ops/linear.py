@@ -132,6 +132,20 @@ class Linear:
             return kernels.gemm_skinny(x, self.weight, None, kernels.EPI_SWIGLU)
         return kernels.swiglu(self(x))
 
+    def clipped_glu(self, x: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
+        """g sigmoid(alpha g) (u + 1) of [gate; up] = x W^T, g = min(gate, limit), u = up clamped to -limit .. limit; with few
+        rows the epilogue of the weight-streaming kernel."""
+        if self.weight.dtype == torch.bfloat16 and self.bias is None and kernels.skinny_ok(x, self.weight):
+            return kernels.gemm_skinny(x, self.weight, None, kernels.EPI_CLIPPED, clip=(limit, alpha))
+        return kernels.clipped_glu(self(x), limit, alpha)
+
+    def gelu_token(self, x: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, col: int) -> torch.Tensor:
+        """gelu_tanh(x W^T) times ``table``[ids, col : col + N]; with few rows the epilogue of the weight-streaming kernel."""
+        if (self.weight.dtype == torch.bfloat16 and table.dtype == torch.bfloat16 and self.bias is None
+                and kernels.skinny_ok(x, self.weight)):
+            return kernels.gemm_skinny(x, self.weight, None, kernels.EPI_GELU_TOKEN, token_rows=(ids, table, col))
+        return kernels.gelu_token(self(x).contiguous(), ids, table, col)
+
     def relu2(self, x: torch.Tensor) -> torch.Tensor:
         """max(x W^T, 0)^2; with few rows the activation is the epilogue of the weight-streaming kernel."""
         if self.weight.dtype == torch.bfloat16 and self.bias is None and kernels.skinny_ok(x, self.weight):
@@ -145,6 +159,18 @@ class Linear:
         if self.weight.dtype == torch.bfloat16 and kernels.skinny_ok(x, self.weight):
             return kernels.gemm_skinny(x, self.weight, self.bias_f32, kernels.EPI_F32_ADD, out=resid)
         return kernels.residual_add(resid, self(x))
+
+    def sums(self, x: torch.Tensor) -> torch.Tensor:
+        """x W^T as a float32 stack [S, T, N] of partial sums (S = 1 where the product is made whole): for a product that
+        becomes the residual stream itself."""
+        if self.weight.dtype == torch.bfloat16 and kernels.skinny_ok(x, self.weight):
+            splits = kernels.skinny_k_splits(self.out_features, self.in_features)
+            y = kernels.gemm_skinny(x, self.weight, self.bias_f32, kernels.EPI_F32, splits)
+            return y if y.dim() == 3 else y.unsqueeze(0)
+        if self.weight.dtype == torch.bfloat16 and self.bias is None and not kernels.skinny_rows(x, self.weight):
+            _library_tuning(x.shape[0])
+            return torch.mm(x, self.weight.t(), out_dtype=torch.float32).unsqueeze(0)
+        return self(x, out_dtype=torch.float32).unsqueeze(0)
 
     def partial(self, x: torch.Tensor) -> torch.Tensor:
         """x W^T as something a norm's ``add_norm`` takes as delta: [T, N], or, when the matrix is

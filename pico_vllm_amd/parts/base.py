@@ -217,8 +217,9 @@ class FeedForward(Part):
 
 class Block(Part):
     """An arrangement of parts.  ``slot_categories`` names its slots and the
-    registry category each is built from."""
+    registry category each is built from; a layer may leave ``optional_slots`` empty."""
     slot_categories: Dict[str, str] = {}
+    optional_slots: tuple = ()
 
     def __init__(self, parts: Dict[str, Part]):
         self.parts = parts
@@ -232,6 +233,11 @@ class Block(Part):
 
     def _sub_parts(self) -> List[Part]:
         return list(self.parts.values())
+
+    def first_norm(self) -> Optional["Norm"]:
+        """The norm through which the layer reads the stream first, if the layer takes its rows from the launch that
+        wrote the stream in front of it (``parts.norm.STREAM_NEXT``)."""
+        return None
 
     @property
     def mixer(self) -> Mixer:

@@ -228,3 +228,55 @@ class PostNormMixerOnlyBlock(PostNormBlock):
     def forward(self, resid, pending, ctx, cache):
         self._mixer(resid, pending, ctx, cache)
         return resid, None
+
+
+@register_part("block", "sandwich_scaled")
+class SandwichBlock(Block):
+    """x += s1 * post1(mixer(norm1(x))); x += s2 * post2(ff(norm2(x))); x += side(x, token): a norm in front of and behind
+    every sublayer, a stored vector on what joins the stream (``scale_names``, behind the layer's prefix), and a layer's own
+    input of the token behind its sublayers.  A layer may leave out the feed-forward (with norm2, post2 and the second
+    vector) and the token input.  The vectors are multiplied into the second norms' weights at load.  Every sum happens in
+    its norm's launch, in float32, and the same launch makes what is read of the new stream next: the next sublayer's norm,
+    the rows the token input reads, or what the next layer reads first (``parts.norm.add_normed``)."""
+    slot_categories = {"norm1": "norm", "mixer": "mixer", "post1": "norm", "norm2": "norm", "ff": "feed_forward", "post2": "norm",
+                       "side": "token_input"}
+    optional_slots = ("norm2", "ff", "post2", "side")
+    graph_safe_prompts = True
+
+    def __init__(self, parts, size: int, scale_names=("ls1", "ls2")):
+        super().__init__(parts)
+        if len({"norm2", "ff", "post2"} & set(parts)) not in (0, 3):
+            raise ValueError("a feed-forward comes with a norm in front of it and one behind it")
+        self.size = int(size)
+        self.scale_names = tuple(scale_names) if "ff" in parts else tuple(scale_names)[:1]
+        self.w1 = self.w2 = None
+
+    def own_param_specs(self):
+        from .spec import ParamSpec
+        return [ParamSpec(n, (self.size,), role="norm") for n in self.scale_names]
+
+    def load_own(self, tensors, device, dtype) -> None:
+        import torch
+        scaled = [(self.parts[p].weight * tensors[n].to(device=device, dtype=torch.float32)).contiguous()
+                  for p, n in zip(("post1", "post2"), self.scale_names)]
+        self.w1, self.w2 = scaled[0], scaled[1] if len(scaled) > 1 else None
+
+    def first_norm(self):
+        from .norm import RMSNorm
+        return self.parts["norm1"] if isinstance(self.parts["norm1"], RMSNorm) else None
+
+    def forward(self, resid, pending, ctx, cache):
+        from .norm import add_normed, take_normed
+        p = self.parts
+        norm1, ff, side = p["norm1"], p.get("ff"), p.get("side")
+        h = take_normed(resid, ctx, norm1) if pending is None else None
+        if h is None:
+            h = norm1.add_norm(resid, pending)
+        after = "rows" if side is not None else None
+        h = add_normed(resid, p["mixer"].forward(h, ctx, cache), self.w1, p["post1"].eps, ctx, norm1.act_dtype,
+                       then=p["norm2"] if ff is not None else after)
+        if ff is not None:
+            h = add_normed(resid, ff.forward(h, ctx), self.w2, p["post2"].eps, ctx, norm1.act_dtype, then=after)
+        if side is not None:
+            add_normed(resid, side.forward(h, ctx), side.norm_weight, side.norm_eps, ctx, norm1.act_dtype)
+        return resid, None

@@ -1,4 +1,4 @@
-"""Dense feed-forwards: SwiGLU, squared ReLU, and none at all."""
+"""Dense feed-forwards: SwiGLU, its clipped form, squared ReLU, and none at all."""
 from __future__ import annotations
 
 from typing import Dict, List, Optional
@@ -42,6 +42,36 @@ class SwiGLUMLP(FeedForward):
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         return self.down.partial(self.gate_up.swiglu(x))
+
+
+@register_part("feed_forward", "clipped_glu_mlp")
+class ClippedGLUMLP(FeedForward):
+    """down( g sigmoid(alpha g) (u + 1) ), g = min(gate x, limit), u = up x clamped to -limit .. limit; no biases.  One
+    product makes gate and up.  ``names``: the three matrices' names behind the part's prefix."""
+    graph_safe_prompts = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, limit: float, alpha: float = 1.702,
+                 names: tuple = ("gate", "up", "down"), act_dtype: torch.dtype = torch.bfloat16):
+        if not limit > 0:
+            raise ValueError(f"the limit must be positive, got {limit}")
+        self.hidden_size, self.intermediate_size, self.limit, self.alpha = hidden_size, intermediate_size, float(limit), float(alpha)
+        self.names = tuple(names)
+        self.gate_up: Optional[Linear] = None
+        self.down: Optional[Linear] = None
+
+    def param_specs(self) -> List[ParamSpec]:
+        H, I = self.hidden_size, self.intermediate_size
+        g, u, d = self.names
+        return [ParamSpec(g, (I, H)), ParamSpec(u, (I, H)), ParamSpec(d, (H, I))]
+
+    def load(self, tensors: Dict[str, torch.Tensor], device, dtype) -> None:
+        g, u = tensors[self.names[0]], tensors[self.names[1]]
+        wdt = torch.float32 if torch.float32 in (g.dtype, u.dtype) else g.dtype
+        self.gate_up = Linear(torch.cat([g.to(wdt), u.to(wdt)], dim=0).to(device))
+        self.down = Linear(tensors[self.names[2]].to(device))
+
+    def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
+        return self.down.partial(self.gate_up.clipped_glu(x, self.limit, self.alpha))
 
 
 @register_part("feed_forward", "relu2_mlp")

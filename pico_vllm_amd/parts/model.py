@@ -9,7 +9,7 @@ from ..config.registry import load_model_description
 from ..ops import kernels
 from ..ops.linear import Linear
 from ..weights.loader import load_checkpoint
-from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, block, delta, gla, latent_attention, mlp, moe, norm, pair, positions, retention, rotary, ssm  # noqa: F401  (register the parts)
+from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, block, delta, gla, input_mix, latent_attention, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401  (register the parts)
 from .base import Block, StepContext
 from .registry import build_part, part_class
 from .spec import CacheSpec, ModelSpec, ParamSpec
@@ -25,11 +25,13 @@ def tensor_name(*pieces: str) -> str:
 
 def _build_layer(lspec, act_dtype) -> Tuple[Block, Dict[str, str]]:
     cls = part_class("block", lspec.block)
-    missing = set(cls.slot_categories) - set(lspec.slots)
+    missing = set(cls.slot_categories) - set(lspec.slots) - set(cls.optional_slots)
     if missing:
         raise ValueError(f"layer {lspec.prefix}: block {lspec.block!r} needs slots {sorted(missing)}")
     parts, sub = {}, {}
     for slot, cat in cls.slot_categories.items():
+        if slot not in lspec.slots:
+            continue
         name, pspec = lspec.slots[slot]
         parts[slot] = build_part(cat, pspec, act_dtype=act_dtype)
         sub[slot] = name
@@ -55,7 +57,7 @@ def model_param_specs(spec: ModelSpec) -> List[ParamSpec]:
     for lspec in spec.layers:
         blk, sub = _build_layer(lspec, torch.float32)
         out += [p for _, _, p in _layer_params(lspec, blk, sub)]
-    for prefix, pspec in tuple(spec.before_layers) + tuple(spec.after_layers):
+    for prefix, pspec in tuple(spec.before_layers) + tuple(spec.after_layers) + ((spec.input_mix,) if spec.input_mix else ()):
         part = build_part("stream", pspec, act_dtype=torch.float32)
         out += [ParamSpec(tensor_name(prefix, p.name), p.shape, p.role, p.std) for p in part.param_specs()]
     fn = build_part("norm", spec.final_norm, act_dtype=torch.float32)
@@ -87,6 +89,10 @@ class DecoderModel:
         # what stands around the layers on the residual stream: (prefix, part)
         self.before = [(pre, build_part("stream", ps, act_dtype=dtype)) for pre, ps in spec.before_layers]
         self.after = [(pre, build_part("stream", ps, act_dtype=dtype)) for pre, ps in spec.after_layers]
+        # what puts the stream and the layers' input together in front of the runs that say so
+        self.mix = [(spec.input_mix[0], build_part("stream", spec.input_mix[1], act_dtype=dtype))] if spec.input_mix else []
+        if not self.mix and any(e.mix_input for e in spec.run_order):
+            raise ValueError("the run order mixes the layers' input in, but the model names no part that does (input_mix)")
         self.embed: Optional[torch.Tensor] = None
         self.head: Optional[Linear] = None
         for i, e in enumerate(spec.run_order):
@@ -137,7 +143,7 @@ class DecoderModel:
                 part.load({p.name: tensors[tensor_name(lspec.prefix, sub[slot], p.name)] for p in part.param_specs()},
                           dev, self.dtype)
             blk.load_own({p.name: tensors[tensor_name(lspec.prefix, p.name)] for p in blk.own_param_specs()}, dev, self.dtype)
-        for prefix, part in self.before + self.after:
+        for prefix, part in self.before + self.after + self.mix:
             part.load({p.name: tensors[tensor_name(prefix, p.name)] for p in part.param_specs()}, dev, self.dtype)
         self.final_norm.load({p.name: tensors[tensor_name(spec.final_norm_name, p.name)]
                               for p in self.final_norm.param_specs()}, dev, self.dtype)
@@ -150,7 +156,7 @@ class DecoderModel:
         return all(p.is_graph_safe(prompts) for p in self._all_parts())
 
     def _all_parts(self):
-        return self.layers + [self.final_norm] + [p for _, p in self.before + self.after]
+        return self.layers + [self.final_norm] + [p for _, p in self.before + self.after + self.mix]
 
     def graph_variant(self, ctx) -> tuple:
         """The host-side choices of all parts for this step, each distinct one once (layers of one kind choose
@@ -167,6 +173,7 @@ class DecoderModel:
         as the run order names it, and the output matrix (the embedding table only as that, when tied)."""
         total = self.head.weight.numel() * self.head.weight.element_size()
         total += sum(self.layers[e.layer].weight_bytes() for e in self.spec.run_order)
+        total += sum(e.mix_input for e in self.spec.run_order) * sum(p.weight_bytes() for _, p in self.mix)
         return total + sum(p.weight_bytes() for _, p in self.before + self.after) + self.final_norm.weight_bytes()
 
     def flops(self, tokens: int, pairs: int, wanted_rows: int) -> float:
@@ -174,6 +181,7 @@ class DecoderModel:
         key) pairs, with logits at ``wanted_rows`` rows: the sum of what the parts report (``Part.flops``)."""
         total = 2.0 * wanted_rows * self.head.weight.numel()
         total += sum(self.layers[e.layer].flops(tokens, pairs) for e in self.spec.run_order)
+        total += sum(e.mix_input for e in self.spec.run_order) * sum(p.flops(tokens, pairs) for _, p in self.mix)
         return total + sum(p.flops(tokens, pairs) for _, p in self.before + self.after)
 
     def forward(self, ctx: StepContext, storage) -> torch.Tensor:
@@ -188,8 +196,18 @@ class DecoderModel:
             resid = self._run_stream(k, part, resid, ctx, storage)
         # runs that take the layers' input again: a copy of the stream as it is now
         entered = resid.clone() if any(e.add_input for e in self.spec.run_order) else None
+        mix = self.mix[0][1] if self.mix else None
+        if mix is not None:
+            mix.enter(resid, ctx)
         pending = None
-        for i, e in enumerate(self.spec.run_order):
+        runs = self.spec.run_order
+        for i, e in enumerate(runs):
+            # what the layer's last launch may leave beside the stream for whoever reads it next
+            after = runs[i + 1] if i + 1 < len(runs) else None
+            ctx.shared[norm.STREAM_NEXT] = (None if after is None or after.add_input else mix.rows(ctx) if after.mix_input
+                                            else self.layers[after.layer].first_norm())
+            if e.mix_input:
+                resid, pending = mix.mix(resid, pending, ctx)
             if e.add_input:
                 kernels.residual_add(resid, entered)       # what is pending joins later; the sums are float32
                 ctx.shared.pop(norm.STREAM_COPY, None)         # a copy of the stream in the activations' dtype is stale now

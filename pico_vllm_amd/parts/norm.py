@@ -13,19 +13,25 @@ from .spec import ParamSpec
 
 @register_part("norm", "rms_norm")
 class RMSNorm(Norm):
-    """y = x / sqrt(mean(x^2) + eps) * weight, in float32 (pico_vllm/RMSNorm.py:22-31)."""
+    """y = x / sqrt(mean(x^2) + eps) * weight, in float32 (pico_vllm/RMSNorm.py:22-31).  ``offset``: what the stored weight is
+    stored around (the weight is offset + stored); ``gain``: a constant on the weight."""
     graph_safe_prompts = True
 
-    def __init__(self, size: int, eps: float, act_dtype: torch.dtype = torch.bfloat16, weight_name: str = "weight"):
+    def __init__(self, size: int, eps: float, act_dtype: torch.dtype = torch.bfloat16, weight_name: str = "weight",
+                 offset: float = 0.0, gain: float = 1.0):
         # weight_name: the gain's name behind the part's prefix; "" where the prefix itself names the tensor
         self.size, self.eps, self.act_dtype, self.weight_name = size, eps, act_dtype, weight_name
+        self.offset, self.gain = float(offset), float(gain)
         self.weight: Optional[torch.Tensor] = None
 
     def param_specs(self) -> List[ParamSpec]:
+        if self.offset:
+            return [ParamSpec(self.weight_name, (self.size,), role="f32", std=0.1)]
         return [ParamSpec(self.weight_name, (self.size,), role="norm")]
 
     def load(self, tensors: Dict[str, torch.Tensor], device, dtype) -> None:
-        self.weight = tensors[self.weight_name].to(device=device, dtype=torch.float32).contiguous()
+        w = tensors[self.weight_name].to(device=device, dtype=torch.float32)
+        self.weight = ((w + self.offset) * self.gain).contiguous() if self.offset or self.gain != 1.0 else w.contiguous()
 
     def add_norm(self, resid, delta, rows=None):
         return kernels.add_rmsnorm(resid, delta, self.weight, self.eps, self.act_dtype, rows)
@@ -85,6 +91,51 @@ def stream_rows(resid: torch.Tensor, ctx, act_dtype: torch.dtype) -> torch.Tenso
     if have is not None and have[0] is resid:
         return have[1]
     return kernels.cast_rows(resid, act_dtype)
+
+
+# What the last launch of a layer leaves beside the stream for whoever reads the stream next.  STREAM_NEXT, set by the
+# model in front of every run: the norm the next layer reads the stream through (``Block.first_norm``), or a ``StreamRows``
+# to be filled with the stream's rows, or None.  STREAM_NORMED, set by the layer that left a norm's rows:
+# (the stream tensor, the norm, its rows).
+STREAM_NEXT, STREAM_NORMED = "stream_next", "stream_normed"
+
+
+class StreamRows:
+    """Room for the stream's rows in the activations' dtype (``rows`` [T, H], row stride free); ``of``: the stream
+    tensor whose rows are in it."""
+
+    def __init__(self, rows: torch.Tensor):
+        self.rows, self.of = rows, None
+
+
+def take_normed(resid: torch.Tensor, ctx, norm: Norm) -> Optional[torch.Tensor]:
+    """The rows of ``norm`` that the launch which last wrote the stream left, if it did."""
+    have = ctx.shared.pop(STREAM_NORMED, None)
+    return have[2] if have is not None and have[0] is resid and have[1] is norm else None
+
+
+def add_normed(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, ctx, act_dtype: torch.dtype,
+               then=None) -> Optional[torch.Tensor]:
+    """resid += rms(y) * weight in one launch that also makes what is read of the new stream next.  ``then``: an RMS norm
+    (its rows are returned), "rows" (the stream's rows in the activations' dtype are returned; in the 32-bit engine the
+    stream itself), or None: the end of the layer, where what ``STREAM_NEXT`` asks for is left."""
+    if then == "rows":
+        if act_dtype == resid.dtype:
+            kernels.norm_add_norm(resid, y, weight, eps)
+            return resid
+        return kernels.norm_add_norm(resid, y, weight, eps, out_dtype=act_dtype)
+    if then is not None:
+        return kernels.norm_add_norm(resid, y, weight, eps, then.weight, then.eps, out_dtype=act_dtype)
+    after = ctx.shared.get(STREAM_NEXT)
+    if isinstance(after, StreamRows):
+        kernels.norm_add_norm(resid, y, weight, eps, out=after.rows)
+        after.of = resid
+    elif isinstance(after, RMSNorm):
+        rows = kernels.norm_add_norm(resid, y, weight, eps, after.weight, after.eps, out_dtype=act_dtype)
+        ctx.shared[STREAM_NORMED] = (resid, after, rows)
+    else:
+        kernels.norm_add_norm(resid, y, weight, eps)
+    return None
 
 
 @register_part("stream", "stream_rms_norm")

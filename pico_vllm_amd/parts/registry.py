@@ -1,6 +1,7 @@
 """Registries: a part kind (a string in a ``PartSpec``) to the class that
 builds it, one registry per category.  A new mixer, feed-forward, norm,
-position encoding, block arrangement or part around the layers ("stream") is added by registering a class; the
+position encoding, block arrangement, part around the layers ("stream") or a layer's own input of the token
+("token_input") is added by registering a class; the
 model builder, the cache manager and the step function only see the
 interfaces in ``parts.base``.
 """
@@ -8,7 +9,7 @@ from __future__ import annotations
 
 from typing import Callable, Dict
 
-CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "stream")
+CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "stream", "token_input")
 _REGISTRY: Dict[str, Dict[str, Callable]] = {c: {} for c in CATEGORIES}
 
 
@@ -26,7 +27,7 @@ def register_part(category: str, kind: str, cls=None):
 def _register_own_parts() -> None:
     """The parts of this package register themselves when their modules load; whoever asks the registry first
     makes sure they have."""
-    from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, block, delta, gla, latent_attention, mlp, moe, norm, pair, positions, retention, rotary, ssm  # noqa: F401
+    from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, block, delta, gla, input_mix, latent_attention, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401
 
 
 def part_class(category: str, kind: str):

@@ -123,6 +123,28 @@ class RotaryPairs(PositionEncoding):
             kernels.rope_pairs_store(x, q_col, 0, 0, self.table(ctx), self.rotary_dim, None, None, None, nq, nkv, dk, dv)
 
 
+class HalvesTable:
+    """Cosines and sines of a step's positions for a rotation whose entry i goes with entry i + rotary_dim / 2 (float32,
+    frequencies as ``scaled_frequencies`` gives them), made once a step for all layers that turn alike."""
+
+    def __init__(self, rotary_dim: int, base: float, scaling=None):
+        self.rotary_dim, self.base = int(rotary_dim), float(base)
+        self.scaling = tuple(float(x) for x in scaling) if scaling else None
+        freqs, self.magnitude = scaled_frequencies(self.rotary_dim, self.base, self.scaling)
+        self._freqs = torch.tensor(freqs, dtype=torch.float64).to(torch.float32)
+        self.inv_freq = None
+
+    def load(self, device) -> None:
+        self.inv_freq = self._freqs.to(device).contiguous()
+
+    def table(self, ctx) -> torch.Tensor:
+        # (a table does not know how the pairs lie, so a rotation of neighbours with the same numbers shares it)
+        key = ("rotary_pairs", self.rotary_dim, self.base, self.scaling)
+        if key not in ctx.shared:
+            ctx.shared[key] = kernels.rope_table(ctx.positions[:ctx.num_tokens], self.inv_freq, self.magnitude)
+        return ctx.shared[key]
+
+
 @register_part("position", "none")
 class NoPosition(PositionEncoding):
     """No position encoding: keys and values are stored as they are."""

@@ -123,10 +123,13 @@ class RunEntry:
     Every entry owns a cache of its own unless ``cache_of`` names an EARLIER
     entry of the run order, whose cache this run's mixer is then given.
     ``add_input``: the residual stream as it entered the first layer (the embeddings with everything
-    ``before_layers`` did to them) is added to the stream in front of this run."""
+    ``before_layers`` did to them) is added to the stream in front of this run.
+    ``mix_input``: the model's ``input_mix`` part makes a new stream out of the stream and that first one in front of
+    this run."""
     layer: int
     cache_of: Optional[int] = None
     add_input: bool = False
+    mix_input: bool = False
 
 
 @dataclass(frozen=True)
@@ -148,6 +151,9 @@ class ModelSpec:
     # learned absolute positions, a norm of the embeddings): (prefix of the part's tensors, the part)
     before_layers: Tuple[Tuple[str, PartSpec], ...] = ()
     after_layers: Tuple[Tuple[str, PartSpec], ...] = ()
+    # what makes a new stream out of the stream and the layers' input in front of the runs that say ``mix_input``
+    # (category "stream"): (prefix of its tensors, the part)
+    input_mix: Optional[Tuple[str, PartSpec]] = None
     embed_scale: float = 1.0          # the embedding rows are multiplied by this (1: as they are)
     logit_softcap: float = 0.0        # > 0: logits = cap * tanh(logits / cap)
     head_bias_name: Optional[str] = None   # a bias [vocab] added to the logits
