@@ -129,6 +129,29 @@ DESIGN_PRESETS.update({
 })
 
 
+def _begasun(vocab, width, layers, heads, kv_heads, dim, rot_dim, kv_rank, ff, side=256) -> Dict:
+    """A Begasun configuration of a real model's proportions, in groups of three layers: attention through a latent, a
+    gated linear recurrence of the model's width, attention over paged keys; every layer with the dense feed-forward and a
+    token input."""
+    lat = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": dim, "kv_rank": kv_rank, "scale": (dim + rot_dim) ** -0.5,
+           "rot": {"dims": rot_dim, "base": 1000000.0, "scaling": {"factor": 4.0, "original": 8192, "fast": 16.0, "slow": 2.0}}}
+    rec = {"width": width, "blocks": heads, "conv": 4}
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+           "rot": {"dims": dim // 2, "base": 1000000.0}}
+    kinds = (("latent_attention", lat), ("rglru", rec), ("attention", att))
+    return {"architecture": "Begasun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5},
+            "logit_scale": 0.5, "token_side": {"dim": side},
+            "layers": [{"type": kinds[i % 3][0], "mixer": kinds[i % 3][1], "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}} for i in range(layers)]}
+
+
+# Begasun at the sizes of the Qwen2.5 shapes: the same width, heads, head size and dense feed-forward; the latent of the
+# Dikolix presets.
+DESIGN_PRESETS.update({
+    "begasun-1.5b": _begasun(151936, 1536, 27, 12, 2, 128, 64, 256, 8960),
+    "begasun-7b": _begasun(152064, 3584, 27, 28, 4, 128, 64, 256, 18944),
+})
+
+
 def preset(name: str) -> Dict:
     import copy
     key = name.lower()
