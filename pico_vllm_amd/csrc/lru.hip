@@ -37,6 +37,25 @@ __device__ __forceinline__ void lru_gate(float zr, float zi, float u, float deca
   add = sqrtf(-expm1f(2.0f * la)) * i * u;
 }
 
+// The same for the chunks' kernels, whose storage is bfloat16: the hardware's exponential (exp2 of the argument times
+// log2 e: a relative error of a few 1e-7) and reciprocal, and 1 - exp(x) for x in -1/2 .. 0 from its Taylor series to the
+// ninth power (the next term is less than 1e-9 of the sum), where 1 - exp(x) itself would lose what is left.
+__device__ __forceinline__ float one_minus_exp(float x) {
+  float p = fmaf(x, 1.0f / 362880, 1.0f / 40320);
+  p = fmaf(p, x, 1.0f / 5040);
+  p = fmaf(p, x, 1.0f / 720);
+  p = fmaf(p, x, 1.0f / 120);
+  p = fmaf(p, x, 1.0f / 24);
+  p = fmaf(p, x, 1.0f / 6);
+  p = fmaf(p, x, 0.5f);
+  p = fmaf(p, x, 1.0f);
+  return x > -0.5f ? -x * p : 1.0f - __expf(x);
+}
+__device__ __forceinline__ void lru_gate_fast(float zr, float zi, float u, float decay, float& la, float& add) {
+  la = decay * __builtin_amdgcn_rcpf(1.0f + __expf(-zr));
+  add = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * la)) * __builtin_amdgcn_rcpf(1.0f + __expf(-zi)) * u;
+}
+
 // V neighbouring outputs of both matrices, summed over one of LRU_SLICES slices of the inner index, two chains an output.
 template <typename T, int V>
 __device__ __forceinline__ void lru_slice_sums(const float* xs, const T* __restrict__ wr, const T* __restrict__ wi, int n, int c,
@@ -79,6 +98,39 @@ __device__ __forceinline__ void lru_slice_sums(const float* xs, const T* __restr
 #pragma unroll
   for (int v = 0; v < V; v++) { sr[v] += r1[v]; si[v] += q1[v]; }
 }
+
+// The same with the rows in registers, two bfloat16 outputs a word, for slices of at most LRU_AHEAD rows: asked for before
+// what they are multiplied with is there.
+#define LRU_AHEAD 16
+struct LruAhead {
+  uint32_t r[LRU_AHEAD], i[LRU_AHEAD];
+  __device__ __forceinline__ void load(const bf16_t* __restrict__ wr, const bf16_t* __restrict__ wi, int n, int c, int slice) {
+    const int i0 = slice * ((n + LRU_SLICES - 1) / LRU_SLICES);
+#pragma unroll
+    for (int k = 0; k < LRU_AHEAD; k++) {
+      const size_t at = (size_t)min(i0 + k, n - 1) * n + c;
+      r[k] = *reinterpret_cast<const uint32_t*>(wr + at);
+      i[k] = *reinterpret_cast<const uint32_t*>(wi + at);
+    }
+  }
+  __device__ __forceinline__ void sums(const float* xs, int n, int slice, float* sr, float* si) const {
+    const int per = (n + LRU_SLICES - 1) / LRU_SLICES, i0 = min(n, slice * per), i1 = min(n, i0 + per);
+    float r1[2] = {0.f, 0.f}, q1[2] = {0.f, 0.f};
+    sr[0] = sr[1] = si[0] = si[1] = 0.f;
+#pragma unroll
+    for (int k = 0; k < LRU_AHEAD; k++) {
+      if (i0 + k < i1) {                                  // even rows to one chain, odd rows to the other, as above
+        const float x = xs[i0 + k];
+        float *a = k & 1 ? r1 : sr, *b = k & 1 ? q1 : si;
+        a[0] = fmaf(x, __uint_as_float(r[k] << 16), a[0]);
+        a[1] = fmaf(x, __uint_as_float(r[k] & 0xffff0000u), a[1]);
+        b[0] = fmaf(x, __uint_as_float(i[k] << 16), b[0]);
+        b[1] = fmaf(x, __uint_as_float(i[k] & 0xffff0000u), b[1]);
+      }
+    }
+    sr[0] += r1[0]; sr[1] += r1[1]; si[0] += q1[0]; si[1] += q1[1];
+  }
+};
 
 __device__ __forceinline__ float lru_slices(const float* part, int width, int c) {
   float s[LRU_SLICES];
@@ -149,9 +201,10 @@ __global__ __launch_bounds__(64) void lru_scan_kernel(const float* __restrict__ 
 
 // One token a sequence.  grid (sequences, blocks): a workgroup owns one part of one sequence, so nobody else reads or
 // writes the history and the state it brings up to date.  x, y: the convolution's inputs and the gate branch in front of
-// its activation, columns of one row each.  TW threads a slice of the inner index, V outputs a thread.
-template <typename T, int V>
-__global__ __launch_bounds__(1024) void lru_step_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ y, int ldy,
+// its activation, columns of one row each.  TW threads a slice of the inner index, V outputs a thread.  AHEAD: parts whose
+// matrices fit the registers of one tile's threads (bfloat16, V 2, n <= LRU_AHEAD x LRU_SLICES, one tile).
+template <typename T, int V, bool AHEAD>
+__global__ __launch_bounds__(AHEAD ? 512 : 1024) void lru_step_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ y, int ldy,
                                                         const float* __restrict__ conv_w, const float* __restrict__ conv_b,
                                                         const T* __restrict__ wr, const T* __restrict__ wi,
                                                         const float* __restrict__ br, const float* __restrict__ bi,
@@ -162,28 +215,44 @@ __global__ __launch_bounds__(1024) void lru_step_kernel(const T* __restrict__ x,
   const int b = blockIdx.x, blk = blockIdx.y, hist = taps - 1;
   const int t = cu_seqlens[b], slot = state_slots[b];
   if (cu_seqlens[b + 1] != t + 1 || slot < 0 || slot >= num_slots) return;      // the whole workgroup alike
+  const int TW = blockDim.x / LRU_SLICES, width = TW * V;
+  const int px = threadIdx.x % TW, slice = threadIdx.x / TW;
+  const T *wrb = wr + (size_t)blk * n * n, *wib = wi + (size_t)blk * n * n;
+  [[maybe_unused]] LruAhead ahead;
+  if constexpr (AHEAD) ahead.load(wrb, wib, n, min(px * V, n - V), slice);
   for (int i = threadIdx.x; i < n; i += blockDim.x) {
     const int c = blk * n + i;
     float* h = state + ((size_t)slot * C + c) * (1 + hist) + 1;
     const float xv = load_f32(x + (size_t)t * ldx + c);
     float acc = conv_b[c];
-    float keep[LRU_MAX_TAPS];
-    for (int j = 0; j < hist; j++) {
-      keep[j] = h[j];
-      acc = fmaf(conv_w[(size_t)j * C + c], keep[j], acc);
+    if (hist <= 3) {                                      // the usual few taps: all of them asked for at once
+      float v[3], w[4];
+#pragma unroll
+      for (int j = 0; j < 4; j++) w[j] = conv_w[(size_t)min(j, hist) * C + c];
+#pragma unroll
+      for (int j = 0; j < 3; j++) v[j] = h[min(j, hist - 1)];       // (no history: the state element in front of it, unused)
+#pragma unroll
+      for (int j = 0; j < 3; j++)
+        if (j < hist) acc = fmaf(w[j], v[j], acc);
+      acc = fmaf(hist == 0 ? w[0] : hist == 1 ? w[1] : hist == 2 ? w[2] : w[3], xv, acc);
+      if (hist > 0) h[hist - 1] = xv;
+      if (hist > 1) h[hist - 2] = hist == 2 ? v[1] : v[2];
+      if (hist > 2) h[0] = v[1];
+    } else {
+      for (int j = 0; j < hist; j++) {
+        const float v = h[j];
+        acc = fmaf(conv_w[(size_t)j * C + c], v, acc);
+        if (j > 0) h[j - 1] = v;
+      }
+      acc = fmaf(conv_w[(size_t)hist * C + c], xv, acc);
+      h[hist - 1] = xv;
     }
-    acc = fmaf(conv_w[(size_t)hist * C + c], xv, acc);
-    for (int j = 0; j + 1 < hist; j++) h[j] = keep[j + 1];
-    if (hist > 0) h[hist - 1] = xv;
     T u;
     store_f32(&u, acc);                                   // as the convolution's own launch leaves it, in the storage type
     xs[i] = load_f32(&u);
   }
   __syncthreads();
-  const int TW = blockDim.x / LRU_SLICES, width = TW * V;
   float* part = xs + n;
-  const int px = threadIdx.x % TW, slice = threadIdx.x / TW;
-  const T *wrb = wr + (size_t)blk * n * n, *wib = wi + (size_t)blk * n * n;
   for (int c0 = 0; c0 < n; c0 += width) {
     // what the last part of the loop needs travels under the products
     const int ce = c0 + (int)threadIdx.x, ch = blk * n + min(ce, n - 1);
@@ -193,7 +262,8 @@ __global__ __launch_bounds__(1024) void lru_step_kernel(const T* __restrict__ x,
     if (mine) { S = *sp; yv = load_f32(y + (size_t)t * ldy + ch); dec = decay[ch]; b_r = br[ch]; b_i = bi[ch]; }
     const int c = c0 + px * V;
     float sr[V], si[V];
-    lru_slice_sums<T, V>(xs, wrb, wib, n, min(c, n - V), slice, sr, si);
+    if constexpr (AHEAD) ahead.sums(xs, n, slice, sr, si);
+    else lru_slice_sums<T, V>(xs, wrb, wib, n, min(c, n - V), slice, sr, si);
     __syncthreads();                                      // the last tile's sums have been read
 #pragma unroll
     for (int v = 0; v < V; v++) {
@@ -242,34 +312,49 @@ __global__ __launch_bounds__(256) void lru_gates_chunk_kernel(const bf16_t* __re
 #pragma unroll
   for (int j = 0; j < 4; j++) zr[j] = zi[j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const u32x4 none = {0u, 0u, 0u, 0u};
-#pragma unroll 2
-  for (int k0 = 0; k0 < n; k0 += 32) {
-    const int k = k0 + 8 * g, ks = min(k, n - 8);          // n is a multiple of 8; behind its end both operands read as zero
-    const bool in = k < n;
-    u32x4 a = *reinterpret_cast<const u32x4*>(arow + ks), r4[4], i4[4];
+  // what the gates read beside their products travels under them
+  float b_r[4], b_i[4], dec[4];
+  bf16_t uv[4][4];
 #pragma unroll
-    for (int j = 0; j < 4; j++) {
-      r4[j] = *reinterpret_cast<const u32x4*>(rrow[j] + ks);
-      i4[j] = *reinterpret_cast<const u32x4*>(irow[j] + ks);
+  for (int j = 0; j < 4; j++) {
+    const int c = min(out0 + 16 * j + i, n - 1), ch = blk * n + c;
+    b_r[j] = br[ch]; b_i[j] = bi[ch]; dec[j] = decay[ch];
+#pragma unroll
+    for (int q = 0; q < 4; q++) uv[j][q] = ub[(size_t)min(t_begin + 16 * wave + 4 * g + q, t_end - 1) * C + c];
+  }
+  for (int k0 = 0; k0 < n; k0 += 64) {                     // two products' operands at a time
+    u32x4 a[2], r4[2][4], i4[2][4];
+#pragma unroll
+    for (int h = 0; h < 2; h++) {
+      const int ks = min(k0 + 32 * h + 8 * g, n - 8);      // n is a multiple of 8; behind its end both operands read as zero
+      a[h] = *reinterpret_cast<const u32x4*>(arow + ks);
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        r4[h][j] = *reinterpret_cast<const u32x4*>(rrow[j] + ks);
+        i4[h][j] = *reinterpret_cast<const u32x4*>(irow[j] + ks);
+      }
     }
-    a = in ? a : none;
 #pragma unroll
-    for (int j = 0; j < 4; j++) {
-      r4[j] = in ? r4[j] : none;
-      i4[j] = in ? i4[j] : none;
-      zr[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, r4[j]), zr[j], 0, 0, 0);
-      zi[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, i4[j]), zi[j], 0, 0, 0);
+    for (int h = 0; h < 2; h++) {
+      const bool in = k0 + 32 * h + 8 * g < n;
+      a[h] = in ? a[h] : none;
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        r4[h][j] = in ? r4[h][j] : none;
+        i4[h][j] = in ? i4[h][j] : none;
+        zr[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a[h]), __builtin_bit_cast(bf16x8, r4[h][j]), zr[j], 0, 0, 0);
+        zi[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a[h]), __builtin_bit_cast(bf16x8, i4[h][j]), zi[j], 0, 0, 0);
+      }
     }
   }
 #pragma unroll
   for (int j = 0; j < 4; j++) {
-    const int c = min(out0 + 16 * j + i, n - 1), ch = blk * n + c;
-    const float b_r = br[ch], b_i = bi[ch], dec = decay[ch];
 #pragma unroll
     for (int q = 0; q < 4; q++) {
-      const int k = 16 * wave + 4 * g + q, t = t_begin + k;
-      float l = 0.f, ad = 0.f;                             // a token behind the chunk's end changes nothing
-      if (t < t_end) lru_gate(zr[j][q] + b_r, zi[j][q] + b_i, bf16_to_f32(ub[(size_t)t * C + c]), dec, l, ad);
+      const int k = 16 * wave + 4 * g + q;
+      float l, ad;
+      lru_gate_fast(zr[j][q] + b_r[j], zi[j][q] + b_i[j], bf16_to_f32(uv[j][q]), dec[j], l, ad);
+      if (t_begin + k >= t_end) l = ad = 0.f;              // a token behind the chunk's end changes nothing
       la[k][16 * j + i] = l;
       add[k][16 * j + i] = ad;
     }
@@ -283,7 +368,7 @@ __global__ __launch_bounds__(256) void lru_gates_chunk_kernel(const bf16_t* __re
   }
 #pragma unroll
   for (int k = 1; k < 16; k++) {
-    s[k] = fmaf(expf(L[k]), s[k - 1], s[k]);
+    s[k] = fmaf(__expf(L[k]), s[k - 1], s[k]);
     L[k] += L[k - 1];
   }
   end_s[wave][lane] = s[15];
@@ -291,7 +376,7 @@ __global__ __launch_bounds__(256) void lru_gates_chunk_kernel(const bf16_t* __re
   __syncthreads();
   float S0 = 0.f, L0 = 0.f;
   for (int v = 0; v < wave; v++) {
-    S0 = fmaf(expf(end_la[v][lane]), S0, end_s[v][lane]);
+    S0 = fmaf(__expf(end_la[v][lane]), S0, end_s[v][lane]);
     L0 += end_la[v][lane];
   }
   const int c = out0 + lane;
@@ -301,12 +386,12 @@ __global__ __launch_bounds__(256) void lru_gates_chunk_kernel(const bf16_t* __re
   for (int k = 0; k < 16; k++) {
     const int t = t_begin + 16 * wave + k;
     if (t < t_end) {
-      local[(size_t)t * C + ch] = fmaf(expf(L[k]), S0, s[k]);
+      local[(size_t)t * C + ch] = fmaf(__expf(L[k]), S0, s[k]);
       sum_la[(size_t)t * C + ch] = L0 + L[k];
     }
   }
   if (wave == 3) {
-    ws_s[(size_t)blockIdx.x * C + ch] = fmaf(expf(L[15]), S0, s[15]);
+    ws_s[(size_t)blockIdx.x * C + ch] = fmaf(__expf(L[15]), S0, s[15]);
     ws_la[(size_t)blockIdx.x * C + ch] = L0 + L[15];
   }
 }
@@ -322,16 +407,16 @@ __global__ __launch_bounds__(64) void lru_combine_kernel(const int* __restrict__
   float* sp = state + ((size_t)slot * C + c) * (1 + hist);
   float S = *sp;
   const int chunks = (n_tok + LRU_CHUNK - 1) / LRU_CHUNK;
-  for (int j0 = 0; j0 < chunks; j0 += 8) {
-    float s[8], l[8];
+  for (int j0 = 0; j0 < chunks; j0 += LRU_TB) {
+    float s[LRU_TB], l[LRU_TB];
 #pragma unroll
-    for (int k = 0; k < 8; k++) {                          // eight chunks' values travel together
+    for (int k = 0; k < LRU_TB; k++) {                     // sixteen chunks' values travel together
       const size_t at = ((size_t)b * max_chunks + min(j0 + k, chunks - 1)) * C + c;
       s[k] = ws_s[at];
       l[k] = ws_la[at];
     }
 #pragma unroll
-    for (int k = 0; k < 8; k++) {
+    for (int k = 0; k < LRU_TB; k++) {
       if (j0 + k >= chunks) break;
       ws_s[((size_t)b * max_chunks + j0 + k) * C + c] = S;
       S = fmaf(expf(l[k]), S, s[k]);
@@ -353,8 +438,8 @@ __global__ __launch_bounds__(256) void lru_chunk_out_kernel(const float* __restr
   const float4 s = *reinterpret_cast<const float4*>(ws_s + ((size_t)b * max_chunks + j) * C + c);
   const bf16_t* yr = y + (size_t)t * ldy + c;
   uint2 o;
-  o.x = pack2_bf16(fmaf(expf(l.x), s.x, h.x) * gelu_tanh_f(bf16_to_f32(yr[0])), fmaf(expf(l.y), s.y, h.y) * gelu_tanh_f(bf16_to_f32(yr[1])));
-  o.y = pack2_bf16(fmaf(expf(l.z), s.z, h.z) * gelu_tanh_f(bf16_to_f32(yr[2])), fmaf(expf(l.w), s.w, h.w) * gelu_tanh_f(bf16_to_f32(yr[3])));
+  o.x = pack2_bf16(fmaf(__expf(l.x), s.x, h.x) * gelu_tanh_f(bf16_to_f32(yr[0])), fmaf(__expf(l.y), s.y, h.y) * gelu_tanh_f(bf16_to_f32(yr[1])));
+  o.y = pack2_bf16(fmaf(__expf(l.z), s.z, h.z) * gelu_tanh_f(bf16_to_f32(yr[2])), fmaf(__expf(l.w), s.w, h.w) * gelu_tanh_f(bf16_to_f32(yr[3])));
   *reinterpret_cast<uint2*>(out + (size_t)t * C + c) = o;
 }
 
@@ -398,14 +483,16 @@ extern "C" int pico_lru_step(const void* x, int ldx, const void* y, int ldy, int
   const int tw = min(128, (units + 7) / 8 * 8);
   const size_t lds = (size_t)(n + 2 * LRU_SLICES * tw * (two ? 2 : 1)) * sizeof(float);
   const dim3 grid(B, blocks);
-#define LAUNCH(TT, V)                                                                                                              \
-  lru_step_kernel<TT, V><<<grid, tw * LRU_SLICES, lds, stream>>>((const TT*)x, ldx, (const TT*)y, ldy, conv_w, conv_b, (const TT*)wr, \
+#define LAUNCH(TT, V, AHEAD)                                                                                                       \
+  lru_step_kernel<TT, V, AHEAD><<<grid, tw * LRU_SLICES, lds, stream>>>((const TT*)x, ldx, (const TT*)y, ldy, conv_w, conv_b, (const TT*)wr, \
                                                                  (const TT*)wi, br, bi, decay, cu_seqlens, state_slots, state,     \
                                                                  num_slots, C, n, taps, (TT*)out)
   if (dtype == PICO_DTYPE_F32) {
-    if (two) LAUNCH(float, 2); else LAUNCH(float, 1);
+    if (two) LAUNCH(float, 2, false); else LAUNCH(float, 1, false);
   } else {
-    if (two) LAUNCH(bf16_t, 2); else LAUNCH(bf16_t, 1);
+    if (two && n <= LRU_AHEAD * LRU_SLICES) LAUNCH(bf16_t, 2, true);       // (one tile of at most 512 threads)
+    else if (two) LAUNCH(bf16_t, 2, false);
+    else LAUNCH(bf16_t, 1, false);
   }
 #undef LAUNCH
   PICO_LAUNCH_CHECK();

@@ -82,6 +82,61 @@ __global__ __launch_bounds__(1024) void qk_norm_store_kernel(
   }
 }
 
+// Unit by unit in bfloat16 for many tokens (one map a head; units of up to 128 entries in whole pairs, the turned ones in
+// whole fours): a lane owns two neighbouring entries, and a wave asks for all of its units (up to QK_AHEAD of them at a time),
+// their partners in the rotation included, before the first norm waits.
+#define QK_AHEAD 4
+__global__ __launch_bounds__(256) void qk_unit_norm_store_kernel(
+    const bf16_t* __restrict__ x, int ld, int q_col, int k_col, int v_col, int nq, int nk, int nv, int dk, int dv,
+    const float* __restrict__ wq, const float* __restrict__ wk, float eps, const float* __restrict__ cos_sin, int rot,
+    const int* __restrict__ slots, bf16_t* __restrict__ q_out, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache, int P,
+    int num_pages) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  const bf16_t* row = x + (size_t)t * ld;
+  const int slot = slots ? slots[t] : -1;
+  const int page = slot >= 0 ? slot / P : -1, off = slot >= 0 ? slot % P : 0;
+  const bool store = page >= 0 && page < num_pages;
+  const int half = rot / 2, i = 2 * lane, ic = min(i, dk - 2);
+  const int j = i < half ? i + half : i < rot ? i - half : ic;        // the partners stand side by side as well
+  float c0 = 1.f, s0 = 0.f, c1 = 1.f, s1 = 0.f;
+  if (i < rot) {
+    const float4 cs = *reinterpret_cast<const float4*>(cos_sin + ((size_t)t * half + (i < half ? i : i - half)) * 2);
+    const float sg = i < half ? -1.f : 1.f;                          // u c - v s in the first half, v c + u s in the second
+    c0 = cs.x; s0 = sg * cs.y; c1 = cs.z; s1 = sg * cs.w;
+  }
+  if (store && v_cache)
+    for (int e = threadIdx.x; e < nv * dv; e += blockDim.x) {
+      const int g = e / dv, d = e % dv;
+      v_cache[(((size_t)page * nv + g) * dv + d) * P + off] = row[v_col + e];
+    }
+  const float2 q0 = *reinterpret_cast<const float2*>(wq + ic), qp = *reinterpret_cast<const float2*>(wq + j);
+  const float2 k0 = *reinterpret_cast<const float2*>(wk + ic), kp = *reinterpret_cast<const float2*>(wk + j);
+  for (int u0 = wave; u0 < nq + nk; u0 += nw * QK_AHEAD) {
+    uint32_t own[QK_AHEAD], par[QK_AHEAD];
+#pragma unroll
+    for (int a = 0; a < QK_AHEAD; a++) {
+      const int u = min(u0 + a * nw, nq + nk - 1);
+      const bf16_t* src = row + (u < nq ? q_col + u * dk : k_col + (u - nq) * dk);
+      own[a] = *reinterpret_cast<const uint32_t*>(src + ic);
+      par[a] = *reinterpret_cast<const uint32_t*>(src + j);
+    }
+#pragma unroll
+    for (int a = 0; a < QK_AHEAD; a++) {
+      const int u = u0 + a * nw;
+      if (u >= nq + nk) break;
+      const bool is_q = u < nq;
+      if (!is_q && !store) break;                                    // (keys stand behind all queries)
+      const float v0 = __uint_as_float(own[a] << 16), v1 = __uint_as_float(own[a] & 0xffff0000u);
+      const float p0 = __uint_as_float(par[a] << 16), p1 = __uint_as_float(par[a] & 0xffff0000u);
+      const float r = 1.0f / sqrtf(wave_sum(i < dk ? fmaf(v0, v0, v1 * v1) : 0.f) / (float)dk + eps);
+      const float2 w0 = is_q ? q0 : k0, w1 = is_q ? qp : kp;
+      const float a0 = v0 * r * w0.x, a1 = v1 * r * w0.y, b0 = p0 * r * w1.x, b1 = p1 * r * w1.y;
+      bf16_t* dst = is_q ? q_out + ((size_t)t * nq + u) * dk : k_cache + (((size_t)page * nk + (u - nq)) * P + off) * dk;
+      if (i < dk) *reinterpret_cast<uint32_t*>(dst + i) = pack2_bf16(a0 * c0 + b0 * s0, a1 * c1 + b1 * s1);
+    }
+  }
+}
+
 extern "C" int pico_qk_norm_store(const void* x, int dtype, int ld, int q_col, int k_col, int v_col, int nq, int nk, int nv,
                                   int dk, int dv, int maps, int norm_mode, const float* wq, const float* wk, float eps,
                                   const float* cos_sin, int rot, const int* slots, void* q_out, void* k_cache, void* v_cache,
@@ -95,6 +150,14 @@ extern "C" int pico_qk_norm_store(const void* x, int dtype, int ld, int q_col, i
   PICO_REQUIRE(k_cache == nullptr || (P > 0 && num_pages > 0 && slots), "pico_qk_norm_store: a cache needs pages and slots");
   if (T == 0) return 0;
   if (k_cache == nullptr) { slots = nullptr; v_cache = nullptr; P = 1; num_pages = 0; }
+  if (dtype == PICO_DTYPE_BF16 && T > 64 && norm_mode == QK_NORM_UNIT && maps == 1 && dk % 2 == 0 && dk <= 128 && rot % 4 == 0 &&
+      (ld | q_col | k_col) % 2 == 0 && ((uintptr_t)x | (uintptr_t)q_out | (uintptr_t)k_cache) % 4 == 0 &&
+      ((uintptr_t)wq | (uintptr_t)wk) % 8 == 0 && (uintptr_t)cos_sin % 16 == 0) {
+    qk_unit_norm_store_kernel<<<T, 256, 0, stream>>>((const bf16_t*)x, ld, q_col, k_col, v_col, nq, nk, nv, dk, dv, wq, wk, eps, cos_sin, rot,
+                                                     slots, (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, P, num_pages);
+    PICO_LAUNCH_CHECK();
+    return 0;
+  }
   // few tokens: a wave a unit, up to sixteen waves, so that a token's units wait for their norms side by side and not one
   // behind the other; many tokens fill the chip with four waves each
   const int threads = T >= 64 ? 256 : 64 * min(16, max(4, nq + nk));

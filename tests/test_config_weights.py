@@ -316,7 +316,7 @@ def test_parts_are_found_by_category_and_kind_and_unknown_ones_are_named():
         register_part("router", "top2")
     with pytest.raises(KeyError, match="no router part"):
         part_class("router", "top2")
-    assert set(CATEGORIES) == {"mixer", "feed_forward", "norm", "position", "block", "stream"}
+    assert set(CATEGORIES) == {"mixer", "feed_forward", "norm", "position", "block", "stream", "token_input"}
 
 
 def test_parts_refuse_sizes_that_make_no_sense_when_they_are_built():

@@ -187,6 +187,38 @@ def conv_rows(x, w, bias, lens, prefix, slots, state, dtype):
                                single=ctx.all_decode, activation="none")
 
 
+@pytest.mark.parametrize("T", [5, 90])
+@pytest.mark.parametrize("H,G,dk,dv,rot", [(12, 2, 128, 128, 64), (3, 1, 24, 40, 8), (8, 2, 64, 32, 64), (1, 1, 64, 16, 0), (5, 5, 10, 12, 4), (2, 2, 32, 32, 2),
+                                           (4, 2, 160, 160, 32)])
+def test_head_norm_rotation_and_store_for_few_and_many_tokens(T, H, G, dk, dv, rot):
+    """bfloat16: units of up to 128 entries of many tokens go two entries a lane; every head of q and of k by itself."""
+    from pico_vllm_amd.ops import kernels
+    g = torch.Generator().manual_seed(H * dk)
+    page, pages = 8, 14
+    cols = (H + G) * dk + G * dv
+    x = rounded(3 * torch.randn(T, cols + (2 if cols % 2 == 0 else 3), generator=g, dtype=F), "bfloat16")
+    wq, wk = 1 + 0.3 * torch.randn(dk, generator=g), 1 + 0.3 * torch.randn(dk, generator=g)
+    pos = torch.arange(40, 40 + T, dtype=torch.int32)
+    slots = torch.tensor([(t * 5) % (page * pages) if t != 4 else -1 for t in range(T)], dtype=torch.int32)
+    table = None
+    if rot:
+        table = kernels.rope_table(pos.to(DEV), torch.tensor(P.frequencies(rot, 300.0)[0], dtype=torch.float32).to(DEV))
+    kc = torch.zeros(pages, G, page, dk, dtype=torch.bfloat16, device=DEV)
+    vc = torch.zeros(pages, G, dv, page, dtype=torch.bfloat16, device=DEV)
+    q = kernels.qk_norm_store(x.to(DEV, torch.bfloat16), 0, H * dk, (H + G) * dk, H, G, G, dk, dv, 1, kernels.QK_NORM_UNIT, wq.to(DEV), wk.to(DEV),
+                              1e-2, table, rot, slots.to(DEV), kc, vc)
+    want_q = P.rotate_half(P.rms(x[:, :H * dk].view(T, H, dk), 1e-2) * wq.to(F), pos, rot, 300.0)
+    want_k = P.rotate_half(P.rms(x[:, H * dk:(H + G) * dk].view(T, G, dk), 1e-2) * wk.to(F), pos, rot, 300.0)
+    close(q.view(T, H, dk), want_q, "bfloat16", scale=0.5)
+    assert float((q.view(T, H, dk).double().cpu() - want_q).abs().mean()) < 2e-3 * float(want_q.abs().mean()) * 2
+    for t, s in enumerate(slots.tolist()):
+        if s >= 0:
+            close(kc[s // page, :, s % page, :], want_k[t], "bfloat16", scale=0.5)
+            assert torch.equal(vc[s // page, :, :, s % page].double().cpu(), x[t, (H + G) * dk:cols].view(G, dv))
+    empty = sorted(set(range(page * pages)) - set(slots.tolist()))
+    assert all(float(kc[s // page, :, s % page, :].float().abs().max()) == 0 for s in empty)
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("C,taps", [(36, 4), (128, 2), (40, 1), (21, 5)])
 def test_the_convolution_without_activation(dtype, C, taps):
