@@ -7,6 +7,7 @@ from . import nasedra as _nasedra  # registers "Nasedra"
 from . import dikolix as _dikolix  # registers "Dikolix"
 from . import vagelix as _vagelix  # registers "Vagelix"
 from . import begasun as _begasun  # registers "Begasun"
+from . import tubusun as _tubusun  # registers "Tubusun"
 from .engine_args import EngineArgs
 
 __all__ = ["ConfigError", "Qwen2Config", "read_config_json", "Architecture", "known_architectures",

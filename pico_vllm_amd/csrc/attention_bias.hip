@@ -10,8 +10,9 @@
 //   sigmoid(gate_i) before it is written
 //   softmax over the visible keys, o_i = sum_j p_ij v_j
 //   instead of a window, chunks: key j <= i is seen iff floor(i / chunk) == floor(j / chunk), chunks counted from
-//   position 0; optionally a sink (a key of score 0 without a value: the softmax's denominator gains a 1); the gate may be
-//   one number a head; several kv heads (of keys) may share one head of values (v_div of them each)
+//   position 0; optionally a sink (a key without a value whose score is 0, or a number a head: the softmax's denominator
+//   gains exp of it); the gate may be one number a head; several kv heads (of keys) may share one head of values (v_div of
+//   them each); optionally a factor on the output, whose rows may lie in a wider buffer
 //
 // A page holds k as [kv heads, page, dk] and v as [kv heads, dv, page].  Scores, softmax and the sums over keys are
 // float32 whatever the storage type.  This file holds the plain kernel (one wave per query token and head, any sizes,
@@ -24,9 +25,12 @@ struct BiasParams {
   float softcap;      // 0: none
   int keep_first;     // with a window: keys below this position are seen whatever their distance
   int chunk;          // > 0: position i sees key j <= i only if floor(i / chunk) == floor(j / chunk) (instead of a window)
-  int sink;           // != 0: one more key of score 0 and no value, p_j = exp(s_j) / (1 + sum exp(s))
+  int sink;           // != 0: one more key without a value, of score 0 or sinks[h]: p_j = exp(s_j) / (exp(sink) + sum exp(s))
   int gate_heads;     // != 0: the gate holds one number a head (gate[t][h]) instead of one an output element
   int v_div;          // kv head g's values are value head g / v_div (several kv heads of keys over one head of values)
+  const float* sinks; // [nq] the sinks' scores (null: 0)
+  float out_scale;    // on the output
+  int out_stride;     // of the output's rows
 };
 
 __device__ __forceinline__ float query_scale(const BiasParams& p, int pos) {
@@ -169,15 +173,17 @@ __global__ __launch_bounds__(64) void attn_bias_plain_kernel(
     for (int i = 0; i < NV; i++) acc[i] = fmaf(acc[i], alpha, blk[i]);
     m = m_new;
   }
-  if (bp.sink) l += expf(-m);                              // the sink's exp(0 - m); the query's own key is always seen
-  T* o = out + ((size_t)t * nq + h) * dv;
+  // the sink's exp(score - m); the query's own key is always seen.  (A sink so far above every key that this overflows
+  // leaves the keys no weight: the output is 0.)
+  if (bp.sink) l += expf((bp.sinks ? bp.sinks[h] : 0.f) - m);
+  T* o = out + (size_t)t * bp.out_stride + (size_t)h * dv;
 #pragma unroll
   for (int i = 0; i < NV; i++) {
     const int dim = lane + 64 * i;
     if (dim >= dv) continue;
-    float v = acc[i] / l;
+    float v = acc[i] / l * bp.out_scale;
     if (gate) v *= 1.0f / (1.0f + expf(-load_f32(gate + (size_t)t * gate_stride + (bp.gate_heads ? (size_t)h : (size_t)h * dv + dim))));
-    if (out32) out32[((size_t)t * nq + h) * dv + dim] = v;
+    if (out32) out32[(size_t)t * bp.out_stride + (size_t)h * dv + dim] = v;
     else store_f32(o + dim, v);
   }
 }
@@ -187,7 +193,8 @@ extern "C" int pico_attn_bias_plain(const void* q, int q_stride, int dtype, cons
                                     void* out, int T, int nq, int nkv, int dk, int dv, int P, int window, float scale,
                                     float temp_coef, int temp_every, float slope_span, int num_pages,
                                     float softcap, int keep_first, const void* gate, int gate_stride, int chunk, int sink,
-                                    int gate_heads, int v_div, int out_f32, hipStream_t stream) {
+                                    int gate_heads, int v_div, int out_f32, const float* sinks, float out_scale, int out_stride,
+                                    hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && nq > 0 && nkv > 0 && dk > 0 && dv > 0 && P > 0 && max_pages > 0 && num_pages > 0,
                "pico_attn_bias_plain: bad sizes");
   PICO_REQUIRE(nq % nkv == 0, "pico_attn_bias_plain: %d query heads are not a multiple of %d kv heads", nq, nkv);
@@ -199,8 +206,9 @@ extern "C" int pico_attn_bias_plain(const void* q, int q_stride, int dtype, cons
   PICO_REQUIRE(gate == nullptr || gate_stride >= (gate_heads ? nq : nq * dv), "pico_attn_bias_plain: gate row stride too small");
   PICO_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "pico_attn_bias_plain: chunks or a window, not both");
   PICO_REQUIRE(v_div >= 1 && nkv % v_div == 0, "pico_attn_bias_plain: %d kv heads do not share values %d each", nkv, v_div);
+  PICO_REQUIRE(out_stride >= nq * dv, "pico_attn_bias_plain: output row stride too small");
   if (T == 0) return 0;
-  const BiasParams bp{scale, temp_coef, slope_span, temp_every, window, softcap, keep_first, chunk, sink, gate_heads, v_div};
+  const BiasParams bp{scale, temp_coef, slope_span, temp_every, window, softcap, keep_first, chunk, sink, gate_heads, v_div, sinks, out_scale, out_stride};
   float* out32 = out_f32 ? (float*)out : nullptr;
   dim3 grid(T, nq);
   const size_t lds = (size_t)(dk + 64) * sizeof(float);

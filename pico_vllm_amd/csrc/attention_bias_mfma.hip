@@ -57,6 +57,10 @@ struct BiasArgs {
   // denominator gains exp(0) (a key of score 0 without a value); gate_heads: the gate holds one number a head;
   // v_div: kv head g reads value head g / v_div; out_f32: `out` is float32
   int chunk, sink, gate_heads, v_div, out_f32;
+  // sinks [nq]: the sinks' scores (null: 0); a factor on the output, and the stride of its rows
+  const float* sinks;
+  float out_scale;
+  int out_stride;
 };
 
 __device__ __forceinline__ float sigmoid_f32(float x) { return 1.0f / (1.0f + __expf(-x)); }
@@ -266,16 +270,18 @@ __global__ __launch_bounds__(256, 2) void attn_bias_kernel(const BiasArgs a) {
     if (kq == 0) { a.parts_ml[2 * c] = M_all; a.parts_ml[2 * c + 1] = L; }
     return;
   }
-  if (a.sink) L += __expf(-M_all);                        // the column's own key is always seen: M_all is finite
-  float inv = 1.0f / L;
+  // the column's own key is always seen: M_all is finite.  (A sink so far above every key that its exponential overflows
+  // leaves the keys no weight: the output is 0.)
+  if (a.sink) L += __expf((a.sinks ? a.sinks[head] : 0.f) - M_all);
+  float inv = a.out_scale / L;
   if (a.gate && a.gate_heads) inv *= sigmoid_f32(bf16_to_f32(a.gate[(size_t)t * a.gate_stride + head]));
-  bf16_t* orow = a.out + ((size_t)t * a.nq + head) * DV + 4 * kq;
+  bf16_t* orow = a.out + (size_t)t * a.out_stride + (size_t)head * DV + 4 * kq;
   const bf16_t* grow = a.gate && !a.gate_heads ? a.gate + (size_t)t * a.gate_stride + (size_t)head * DV + 4 * kq : nullptr;
 #pragma unroll
   for (int tt = 0; tt < DT; tt++) {
     float g0 = inv, g1 = inv, g2 = inv, g3 = inv;
     if (a.out_f32) {
-      float* o32 = reinterpret_cast<float*>(a.out) + ((size_t)t * a.nq + head) * DV + 4 * kq + 16 * tt;
+      float* o32 = reinterpret_cast<float*>(a.out) + (size_t)t * a.out_stride + (size_t)head * DV + 4 * kq + 16 * tt;
       *reinterpret_cast<f32x4*>(o32) = f32x4{o[tt][0] * g0, o[tt][1] * g1, o[tt][2] * g2, o[tt][3] * g3};
       continue;
     }
@@ -297,7 +303,8 @@ __global__ __launch_bounds__(256, 2) void attn_bias_kernel(const BiasArgs a) {
 // The pieces of a column's keys put together: out = sum_z o_z e^(m_z - M) / sum_z l_z e^(m_z - M), z in ascending order.
 __global__ __launch_bounds__(DV <= 64 ? 64 : DV <= 128 ? 128 : 256) void attn_bias_merge_kernel(
     const float* __restrict__ parts_o, const float* __restrict__ parts_ml, int chunks, int ncols, bf16_t* __restrict__ out,
-    const bf16_t* __restrict__ gate, int gate_stride, int nq, int sink, int gate_heads, int out_f32) {
+    const bf16_t* __restrict__ gate, int gate_stride, int nq, int sink, int gate_heads, int out_f32, const float* __restrict__ sinks,
+    float out_scale, int out_stride) {
   // the pieces' maxima and sums once into LDS (one load a thread, all in flight together), then every thread its sum
   __shared__ float ms[MAX_PIECES], ws[MAX_PIECES];
   const int c = blockIdx.x, d = threadIdx.x;
@@ -317,11 +324,12 @@ __global__ __launch_bounds__(DV <= 64 ? 64 : DV <= 128 ? 128 : 256) void attn_bi
     L += ws[z] * w;
     acc += parts_o[((size_t)z * ncols + c) * DV + d] * w;
   }
-  if (sink) L += __expf(-M);
-  float v = acc / L;
+  if (sink) L += __expf((sinks ? sinks[c % nq] : 0.f) - M);
+  float v = acc / L * out_scale;
   if (gate) v *= sigmoid_f32(bf16_to_f32(gate[(size_t)(c / nq) * gate_stride + (gate_heads ? (size_t)(c % nq) : (size_t)(c % nq) * DV + d)]));
-  if (out_f32) reinterpret_cast<float*>(out)[(size_t)c * DV + d] = v;
-  else out[(size_t)c * DV + d] = f32_to_bf16(v);
+  const size_t at = (size_t)(c / nq) * out_stride + (size_t)(c % nq) * DV + d;
+  if (out_f32) reinterpret_cast<float*>(out)[at] = v;
+  else out[at] = f32_to_bf16(v);
 }
 
 // split != 0: one block of 16 columns a workgroup, its keys shared by the four waves; else four blocks a workgroup.
@@ -330,7 +338,8 @@ extern "C" int pico_attnb(const void* q, int q_stride, const void* k_cache, cons
                           int nq, int nkv, int dk, int dv, int P, int num_pages, float scale, int window, float temp_coef,
                           int temp_every, float slope_span, int split, int chunks, float* parts_o, float* parts_ml,
                           float softcap, int keep_first, const void* gate, int gate_stride, int chunk, int sink,
-                          int gate_heads, int v_div, int out_f32, hipStream_t stream) {
+                          int gate_heads, int v_div, int out_f32, const float* sinks, float out_scale, int out_stride,
+                          hipStream_t stream) {
   PICO_REQUIRE(dk == DK && dv == DV, "pico_attnb: built for keys of %d and values of %d, asked for %d and %d", DK, DV, dk, dv);
   PICO_REQUIRE(T >= 0 && num_seqs > 0 && nq > 0 && nkv > 0 && nq % nkv == 0 && max_pages > 0 && num_pages > 0,
                "pico_attnb: bad sizes");
@@ -343,6 +352,8 @@ extern "C" int pico_attnb(const void* q, int q_stride, const void* k_cache, cons
   PICO_REQUIRE(gate == nullptr || (gate_heads ? gate_stride >= nq : (gate_stride >= nq * DV && gate_stride % 4 == 0 && (uintptr_t)gate % 8 == 0)),
                "pico_attnb: gate rows must be 8-byte aligned and hold all heads");
   PICO_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "pico_attnb: chunks or a window, not both");
+  PICO_REQUIRE(out_stride >= nq * DV && out_stride % 4 == 0 && (uintptr_t)out % (out_f32 ? 16 : 8) == 0,
+               "pico_attnb: output rows of %d must hold all heads and start on four entries", out_stride);
   PICO_REQUIRE(v_div >= 1 && nkv % v_div == 0, "pico_attnb: %d kv heads do not share values %d each", nkv, v_div);
   if (T == 0) return 0;
   const int R = nq / nkv;
@@ -353,13 +364,14 @@ extern "C" int pico_attnb(const void* q, int q_stride, const void* k_cache, cons
   BiasArgs a{(const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, max_pages,
              cu_seqlens, positions, (bf16_t*)out, num_seqs, nq, nkv, P, num_pages, window, temp_every, scale, temp_coef,
              slope_span, chunks, T * nq, parts_o, parts_ml, softcap, keep_first, (const bf16_t*)gate, gate_stride,
-             chunk, sink, gate_heads, v_div, out_f32};
+             chunk, sink, gate_heads, v_div, out_f32, sinks, out_scale, out_stride};
   if (split) {
     attn_bias_kernel<true><<<dim3((unsigned)tiles, nkv, chunks), 256, 0, stream>>>(a);
     if (chunks > 1)
       attn_bias_merge_kernel<<<T * nq, DV <= 64 ? 64 : DV <= 128 ? 128 : 256, 0, stream>>>(parts_o, parts_ml, chunks, T * nq,
                                                                                            (bf16_t*)out, (const bf16_t*)gate,
-                                                                                           gate_stride, nq, sink, gate_heads, out_f32);
+                                                                                           gate_stride, nq, sink, gate_heads, out_f32, sinks,
+                                                                                           out_scale, out_stride);
   } else
     attn_bias_kernel<false><<<dim3((unsigned)((tiles + 3) / 4), nkv), 256, 0, stream>>>(a);
   PICO_LAUNCH_CHECK();

@@ -56,6 +56,12 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return z / (1.0f + expf(-2.0f * a));
 }
 
+// 0.5 z (1 + erf(z / sqrt 2))
+__device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)); }
+
+// z sigmoid(z)
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+
 // A value combined with the one 16 (32) lanes across, in both lanes: one vector instruction of gfx950
 // (v_permlane16_swap / v_permlane32_swap give both values in two registers) where an exchange through the LDS crossbar
 // (what __shfl_xor compiles to) waits in line behind the tiles' reads.  Maximum and sum are symmetric, so both lanes

@@ -6,29 +6,29 @@
 #include "common.h"
 
 // ---------------------------------------------------------------------------
-// embedding: out[t, :] = table[ids[t], :] * scale as float32.  An id outside [0, V) gives a
+// embedding: out[t, :] = table[ids[t], :] * scale (+ vec, the same vector for every row) as float32.  An id outside [0, V) gives a
 // row of zeros (the host checks ids before a step; this only keeps the kernel in bounds).
 // Reference: nn.Embedding lookup, pico_vllm/model.py:427.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void embedding_kernel(const T* __restrict__ table, const int* __restrict__ ids,
-                                 float* __restrict__ out, int H, int V, float scale) {
+                                 float* __restrict__ out, int H, int V, float scale, const float* __restrict__ vec) {
   const int t = blockIdx.x;
   const int id = ids[t];
   const bool ok = id >= 0 && id < V;
   const T* row = table + (size_t)(ok ? id : 0) * H;
   float* o = out + (size_t)t * H;
-  for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = ok ? load_f32(row + i) * scale : 0.f;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = (ok ? load_f32(row + i) * scale : 0.f) + (vec ? vec[i] : 0.f);
 }
 
 extern "C" int pico_embedding(const void* table, int table_dtype, const int* ids, float* out, int T, int H,
-                              int V, float scale, hipStream_t stream) {
+                              int V, float scale, const float* vec, hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && H > 0 && V > 0, "pico_embedding: bad sizes T=%d H=%d V=%d", T, H, V);
   if (T == 0) return 0;
   if (table_dtype == PICO_DTYPE_F32)
-    embedding_kernel<float><<<T, 256, 0, stream>>>((const float*)table, ids, out, H, V, scale);
+    embedding_kernel<float><<<T, 256, 0, stream>>>((const float*)table, ids, out, H, V, scale, vec);
   else if (table_dtype == PICO_DTYPE_BF16)
-    embedding_kernel<bf16_t><<<T, 256, 0, stream>>>((const bf16_t*)table, ids, out, H, V, scale);
+    embedding_kernel<bf16_t><<<T, 256, 0, stream>>>((const bf16_t*)table, ids, out, H, V, scale, vec);
   else
     PICO_REQUIRE(false, "pico_embedding: unknown dtype %d", table_dtype);
   PICO_LAUNCH_CHECK();
@@ -634,44 +634,71 @@ extern "C" int pico_add_rows(float* resid, const void* table, int table_dtype, c
   return 0;
 }
 
-// ---------------------------------------------------------------------------
-// Squared ReLU: out = max(x, 0)^2, element by element (in place when out == x).
-// ---------------------------------------------------------------------------
-template <typename T>
-__global__ void relu2_kernel(const T* __restrict__ x, T* __restrict__ out, size_t n) {
-  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < n) {
-    const float v = fmaxf(load_f32(x + i), 0.f);
-    store_f32(out + i, v * v);
-  }
+// resid[t, :] += vec[:] in float32
+__global__ __launch_bounds__(256) void add_vector_kernel(float* __restrict__ resid, const float* __restrict__ vec, int H) {
+  for (int i = threadIdx.x; i < H; i += blockDim.x) resid[(size_t)blockIdx.x * H + i] += vec[i];
 }
 
-__global__ void relu2_bf16x8_kernel(const uint4* __restrict__ x, uint4* __restrict__ out, size_t n8) {
+extern "C" int pico_add_vector(float* resid, const float* vec, int T, int H, hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && H > 0, "pico_add_vector: bad sizes");
+  if (T == 0) return 0;
+  add_vector_kernel<<<T, 256, 0, stream>>>(resid, vec, H);
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------
+// Activations element by element (in place when out == x): squared ReLU max(x, 0)^2, gelu with the error function.
+// ---------------------------------------------------------------------------
+#define ACT_RELU2 0
+#define ACT_GELU 1
+template <int ACT> __device__ __forceinline__ float act_of(float v) {
+  if (ACT == ACT_GELU) return gelu_erf_f(v);
+  v = fmaxf(v, 0.f);
+  return v * v;
+}
+
+template <typename T, int ACT>
+__global__ void act_kernel(const T* x, T* out, size_t n) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) store_f32(out + i, act_of<ACT>(load_f32(x + i)));
+}
+
+template <int ACT>
+__global__ void act_bf16x8_kernel(const uint4* x, uint4* out, size_t n8) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n8) return;
   uint4 v = x[i];
   uint32_t* w = reinterpret_cast<uint32_t*>(&v);
 #pragma unroll
   for (int j = 0; j < 4; j++) {
-    const float a = fmaxf(__uint_as_float(w[j] << 16), 0.f), b = fmaxf(__uint_as_float(w[j] & 0xffff0000u), 0.f);
-    w[j] = pack2_bf16(a * a, b * b);
+    w[j] = pack2_bf16(act_of<ACT>(__uint_as_float(w[j] << 16)), act_of<ACT>(__uint_as_float(w[j] & 0xffff0000u)));
   }
   out[i] = v;
 }
 
-extern "C" int pico_relu2(const void* x, void* out, int dtype, long long n, hipStream_t stream) {
-  PICO_REQUIRE(n >= 0, "pico_relu2: bad size");
+template <int ACT>
+static int act_launch(const void* x, void* out, int dtype, long long n, const char* who, hipStream_t stream) {
+  PICO_REQUIRE(n >= 0, "%s: bad size", who);
   if (n == 0) return 0;
   if (dtype == PICO_DTYPE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0) {
     const size_t n8 = (size_t)n / 8;
-    relu2_bf16x8_kernel<<<(unsigned)((n8 + 255) / 256), 256, 0, stream>>>((const uint4*)x, (uint4*)out, n8);
+    act_bf16x8_kernel<ACT><<<(unsigned)((n8 + 255) / 256), 256, 0, stream>>>((const uint4*)x, (uint4*)out, n8);
   } else if (dtype == PICO_DTYPE_BF16) {
-    relu2_kernel<bf16_t><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, (size_t)n);
+    act_kernel<bf16_t, ACT><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, (size_t)n);
   } else if (dtype == PICO_DTYPE_F32) {
-    relu2_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>((const float*)x, (float*)out, (size_t)n);
+    act_kernel<float, ACT><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>((const float*)x, (float*)out, (size_t)n);
   } else {
-    PICO_REQUIRE(false, "pico_relu2: unknown dtype %d", dtype);
+    PICO_REQUIRE(false, "%s: unknown dtype %d", who, dtype);
   }
   PICO_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int pico_relu2(const void* x, void* out, int dtype, long long n, hipStream_t stream) {
+  return act_launch<ACT_RELU2>(x, out, dtype, n, "pico_relu2", stream);
+}
+
+extern "C" int pico_gelu(const void* x, void* out, int dtype, long long n, hipStream_t stream) {
+  return act_launch<ACT_GELU>(x, out, dtype, n, "pico_gelu", stream);
 }

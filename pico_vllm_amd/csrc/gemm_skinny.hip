@@ -56,6 +56,7 @@ struct TileRows {
 #define EPI_CLIPPED 5  // W = [gate rows; up rows], out bf16 [M, N / 2] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up
                        // clamped to -limit .. limit
 #define EPI_GELU_TOKEN 6   // out bf16 [M, N] = gelu_tanh(x W^T + bias) times columns of a table's row of the token
+#define EPI_GELU 7     // out bf16 [M, N] = gelu(x W^T + bias), with the error function
 #define MAX_SK_SLABS 8 // partial sums that a norm in front of a projection adds up
 
 // W's rows come in pairs (gate, up) whose sums meet in one output
@@ -364,6 +365,7 @@ __device__ __forceinline__ void skinny_finish(float (*red)[MT][16][64], int tile
           v[b] = fmaxf(v[b], 0.f);
           v[b] *= v[b];
         }
+        if (EPI == EPI_GELU) v[b] = gelu_erf_f(v[b]);
       }
       if (EPI == EPI_GELU_TOKEN) {
         const bf16_t* e = ex.table + (size_t)min(max(ex.ids[m], 0), ex.rows - 1) * ex.ld;
@@ -689,7 +691,7 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   PICO_REQUIRE(K % 8 == 0 && ldx % 8 == 0 && ldw % 8 == 0 && ldx >= K && ldw >= K,
                "pico_gemm_skinny: K and the row strides must be multiples of 8 (K=%d ldx=%d ldw=%d)", K, ldx, ldw);
   PICO_REQUIRE((uintptr_t)X % 16 == 0 && (uintptr_t)W % 16 == 0, "pico_gemm_skinny: operands must be 16-byte aligned");
-  PICO_REQUIRE(epilogue >= 0 && epilogue <= 6, "pico_gemm_skinny: unknown epilogue %d", epilogue);
+  PICO_REQUIRE(epilogue >= 0 && epilogue <= 7, "pico_gemm_skinny: unknown epilogue %d", epilogue);
   PICO_REQUIRE(k_splits >= 1 && (k_splits == 1 || epilogue == EPI_F32), "pico_gemm_skinny: only the float32 epilogue can split k over the grid");
   PICO_REQUIRE(!sk_paired(epilogue) || (N % 2 == 0 && bias == nullptr), "pico_gemm_skinny: gated activations need an even N and no bias");
   PICO_REQUIRE(epilogue != EPI_CLIPPED || limit > 0.f, "pico_gemm_skinny: the clipped activation needs a positive limit");
@@ -727,6 +729,7 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
     else if (epilogue == EPI_F32_ADD) LAUNCHP(EPI_F32_ADD);
     else if (epilogue == EPI_CLIPPED) LAUNCHP(EPI_CLIPPED);
     else if (epilogue == EPI_GELU_TOKEN) LAUNCHP(EPI_GELU_TOKEN);
+    else if (epilogue == EPI_GELU) LAUNCHP(EPI_GELU);
     else LAUNCHP(EPI_SWIGLU);
 #undef LAUNCHP
     PICO_LAUNCH_CHECK();
@@ -761,6 +764,7 @@ extern "C" int pico_gemm_skinny(const void* X, int ldx, const void* W, int ldw, 
   else if (epilogue == EPI_F32_ADD) LAUNCH(EPI_F32_ADD);
   else if (epilogue == EPI_CLIPPED) LAUNCH(EPI_CLIPPED);
   else if (epilogue == EPI_GELU_TOKEN) LAUNCH(EPI_GELU_TOKEN);
+  else if (epilogue == EPI_GELU) LAUNCH(EPI_GELU);
   else LAUNCH(EPI_SWIGLU);
 #undef LAUNCH4
 #undef LAUNCH

@@ -5,6 +5,8 @@
 //     o_t[v]    = sum_c S_t[c][v] * q_t[c] * qscale
 //   alpha_t = sigmoid(z_t)^(1 / tau),  z_t = A2 (A1 h_t) + b           (a low-rank projection; A1 h_t comes with q, k, v)
 //   out_t = rmsnorm_v(o_t) * w * silu(g_t)                             (every head by itself, one weight for all heads)
+//   or out_t = rmsnorm(o_t) * w * sigmoid(g_t) with all heads of a token as one row (pico_gated_row_norm)
+// Optionally q, k and v go through z sigmoid(z) as they are read, and a head's decay is a constant.
 //
 // The state lives in float32, one [heads, dk, dv] block per state slot; decays, their logarithms, the recurrence and
 // the head norm are float32 whatever the storage type T of the projections.  Every sum runs in an order that depends
@@ -79,7 +81,7 @@ __global__ __launch_bounds__(TB == 16 ? 256 : 512) void gla_scan_kernel(const T*
                                                        int num_slots, int chunk, int max_chunks, float* __restrict__ ws,
                                                        float* __restrict__ ws_decay, const T* __restrict__ a2,
                                                        const float* __restrict__ a2_bias, int a_col, int R, float inv_tau,
-                                                       const float* __restrict__ head_decay) {
+                                                       const float* __restrict__ head_decay, int silu) {
   extern __shared__ float lds[];
   // head_decay given: every key channel of head h decays by the constant head_decay[h] at every token (log_decay, a2
   // are not read); the decay is multiplied in as it is, no logarithm and exponential between
@@ -179,15 +181,19 @@ __global__ __launch_bounds__(TB == 16 ? 256 : 512) void gla_scan_kernel(const T*
     for (int j = 0; j < NL; j++) {
       const int tt = tt0 + 2 * j, c = cc, i = tt * CP + c;      // = threadIdx.x + j * blockDim.x: a workgroup has 2 CP threads
       const bool in = tt < nb && c < dk;
-      qs[i] = (in && MODE != GLA_LOCAL) ? load_f32(&rq[j]) * qscale : 0.f;
-      ks[i] = in ? load_f32(&rk[j]) : 0.f;
+      const float qv = load_f32(&rq[j]), kv = load_f32(&rk[j]);
+      qs[i] = (in && MODE != GLA_LOCAL) ? (silu ? silu_f(qv) : qv) * qscale : 0.f;
+      ks[i] = in ? (silu ? silu_f(kv) : kv) : 0.f;
       as[i] = in ? (head_decay ? fixed : expf(ra[j])) : 1.f;
     }
     float vv[VPL][TB];
 #pragma unroll
     for (int j = 0; j < VPL; j++)
 #pragma unroll
-      for (int tt = 0; tt < TB; tt++) vv[j][tt] = (tt < nb && v_ok[j]) ? load_f32(&rv[j][tt]) : 0.f;
+      for (int tt = 0; tt < TB; tt++) {
+        const float x0 = load_f32(&rv[j][tt]);
+        vv[j][tt] = (tt < nb && v_ok[j]) ? (silu ? silu_f(x0) : x0) : 0.f;
+      }
     __syncthreads();
     if (t0 + TB < t_end) fetch(t0 + TB);
 #pragma unroll
@@ -277,7 +283,7 @@ extern "C" int pico_gla_scan(const void* x, int ldx, int dtype, int q_col, int k
                              const int* cu_seqlens, const int* state_slots, float* state, float* out, int num_seqs,
                              int T, int H, int dk, int dv, float qscale, int num_slots, int chunk, int max_chunks,
                              float* ws, float* ws_decay, const void* a2, const float* a2_bias, int a_col, int R, float tau,
-                             const float* head_decay, hipStream_t stream) {
+                             const float* head_decay, int silu, hipStream_t stream) {
   PICO_REQUIRE(head_decay != nullptr || log_decay != nullptr || (chunk == 0 && a2 != nullptr && R > 0 && a_col >= 0 && ldx >= a_col + R && tau > 0.f),
                "pico_gla_scan: without the decays' logarithms the walk needs what makes them, and runs whole");
   PICO_REQUIRE(num_seqs >= 0 && T >= 0 && H > 0 && dk > 0 && dv > 0 && num_slots > 0, "pico_gla_scan: bad sizes");
@@ -301,7 +307,7 @@ extern "C" int pico_gla_scan(const void* x, int ldx, int dtype, int q_col, int k
   const int vb = (dv + 64 * vpl - 1) / (64 * vpl);
 #define GLA_ARGS(TT)                                                                                                       \
   (const TT*)x, ldx, q_col, k_col, v_col, log_decay, cu_seqlens, state_slots, state, out, H, dk, dv, qscale, num_slots,   \
-      chunk, max_chunks, ws, ws_decay, (const TT*)a2, a2_bias, a_col, R, 1.0f / (tau > 0.f ? tau : 1.f), head_decay
+      chunk, max_chunks, ws, ws_decay, (const TT*)a2, a2_bias, a_col, R, 1.0f / (tau > 0.f ? tau : 1.f), head_decay, silu
 #define GLA_LAUNCH(TT, MODE, GX)                                                                                           \
   do {                                                                                                                     \
     constexpr bool fused = MODE == GLA_WHOLE;     /* with FUSED the launch below is taken only when log_decay is null */ \
@@ -377,6 +383,55 @@ extern "C" int pico_gla_out(const float* o, const void* g, int ldg, int dtype, c
     gla_out_kernel<bf16_t><<<grid, 64, 0, stream>>>(o, (const bf16_t*)g, ldg, w, eps, (bf16_t*)out, H, dv, sigmoid_gate);
   else
     PICO_REQUIRE(false, "pico_gla_out: unknown dtype %d", dtype);
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------
+// Norm over all heads of a token at once, and gate: out[t][i] = o[t][i] / sqrt(mean_i(o^2) + eps) * w[i] * sigmoid(g[t][i]).
+// o float32 [T, N]; g: columns of a wider row of type T (stride ldg); out rows of type T (stride ldo).  One workgroup a
+// token, its row in registers: thread i owns entries i, i + blockDim, ..; the number of threads goes with N alone.
+// ---------------------------------------------------------------------------
+#define ROW_NORM_VPT 8
+template <typename T>
+__global__ __launch_bounds__(1024) void gated_row_norm_kernel(const float* __restrict__ o, const T* __restrict__ g, int ldg,
+                                                              const float* __restrict__ w, float eps, T* __restrict__ out,
+                                                              int ldo, int N) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  float v[ROW_NORM_VPT], gv[ROW_NORM_VPT], wv[ROW_NORM_VPT];
+#pragma unroll
+  for (int j = 0; j < ROW_NORM_VPT; j++) {
+    if (j * (int)blockDim.x >= N) break;
+    const int i = min(j * (int)blockDim.x + (int)threadIdx.x, N - 1);
+    v[j] = o[(size_t)t * N + i];
+    gv[j] = load_f32(g + (size_t)t * ldg + i);
+    wv[j] = w[i];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < ROW_NORM_VPT; j++)
+    if (j * (int)blockDim.x + (int)threadIdx.x < N) ss = fmaf(v[j], v[j], ss);
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / (float)N + eps);
+#pragma unroll
+  for (int j = 0; j < ROW_NORM_VPT; j++) {
+    const int i = j * (int)blockDim.x + (int)threadIdx.x;
+    if (i < N) store_f32(out + (size_t)t * ldo + i, v[j] * r * wv[j] / (1.0f + expf(-gv[j])));
+  }
+}
+
+extern "C" int pico_gated_row_norm(const float* o, const void* g, int ldg, int dtype, const float* w, float eps, void* out,
+                                   int ldo, int T, int N, hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && N > 0 && ldg >= N && ldo >= N && eps > 0.f, "pico_gated_row_norm: bad sizes");
+  PICO_REQUIRE(N <= 1024 * ROW_NORM_VPT, "pico_gated_row_norm: rows of at most %d entries, got %d", 1024 * ROW_NORM_VPT, N);
+  if (T == 0) return 0;
+  const int threads = N <= 256 ? 64 : N <= 2048 ? 256 : 1024;
+  if (dtype == PICO_DTYPE_F32)
+    gated_row_norm_kernel<float><<<T, threads, 0, stream>>>(o, (const float*)g, ldg, w, eps, (float*)out, ldo, N);
+  else if (dtype == PICO_DTYPE_BF16)
+    gated_row_norm_kernel<bf16_t><<<T, threads, 0, stream>>>(o, (const bf16_t*)g, ldg, w, eps, (bf16_t*)out, ldo, N);
+  else
+    PICO_REQUIRE(false, "pico_gated_row_norm: unknown dtype %d", dtype);
   PICO_LAUNCH_CHECK();
   return 0;
 }

@@ -11,6 +11,8 @@
 // Wd_e (silu(Wg_e x) * (Wu_e x)) and the weight scales its OUTPUT (here: y, in front of the linear Wd_e); router outputs
 // from E on stand for experts that hand their input on unchanged.
 //
+// A third (MOE_MODE_CLIPPED_OUT): the experts of the first family with the weight on the OUTPUT (here: on y, as above).
+//
 // Expert matrices are stacked: gate_up [E, 2 F, D] (an expert's gate rows, then its up rows), down [E, D, F].
 // This file holds the plain kernels (one wave per output element, any sizes, float32 or bfloat16 storage, every sum
 // in float32 and in an order that depends on the sizes alone); the matrix-core kernels for many rows stand behind them.
@@ -165,13 +167,15 @@ extern "C" int pico_moe_route(const float* logits, int T, int E, int top, int* e
 
 #define MOE_MODE_CLIPPED 0
 #define MOE_MODE_SOFTMAX_SWIGLU 1
+#define MOE_MODE_CLIPPED_OUT 2
 
-// mode 0: the clipped activation, the row's weight w already in the input; mode 1: w silu(g) u
+// mode 0: the clipped activation, the row's weight w already in the input; mode 1: w silu(g) u; mode 2: w times the clipped
+// activation
 __device__ __forceinline__ float expert_act(float g, float u, float limit, float alpha, int mode, float w) {
   if (mode == MOE_MODE_SOFTMAX_SWIGLU) return w * (g / (1.0f + expf(-g))) * u;
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+  return (mode == MOE_MODE_CLIPPED_OUT ? w : 1.0f) * (g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
 }
 
 // ---------------------------------------------------------------------------
@@ -283,7 +287,7 @@ __global__ __launch_bounds__(256) void moe_up_plain_kernel(const T* __restrict__
   const int e = experts[r];
   if (e < 0 || e >= E) return;
   const float wr = weights[r];
-  const float w = mode == MOE_MODE_SOFTMAX_SWIGLU ? 1.f : wr;
+  const float w = mode != MOE_MODE_CLIPPED ? 1.f : wr;
   const T* x = h + (size_t)(r / top) * ldh;
   const T* We = gate_up + (size_t)e * 2 * F * D;
   for (int i = 0; i < 4; i++) {
@@ -293,7 +297,7 @@ __global__ __launch_bounds__(256) void moe_up_plain_kernel(const T* __restrict__
     const T* wu = We + (size_t)(F + f) * D;
     float g = 0.f, u = 0.f;
     for (int j = lane; j < D; j += 64) {
-      const float xv = mode == MOE_MODE_SOFTMAX_SWIGLU ? load_f32(x + j) : scaled_input<T>(x + j, w);
+      const float xv = mode != MOE_MODE_CLIPPED ? load_f32(x + j) : scaled_input<T>(x + j, w);
       g = fmaf(load_f32(wg + j), xv, g);
       u = fmaf(load_f32(wu + j), xv, u);
     }
@@ -333,7 +337,7 @@ extern "C" int pico_moe_experts_plain(const void* h, int ldh, int dtype, const v
                                       const int* experts, const float* weights, void* y, float* out, int T, int top,
                                       int E, int F, int D, float limit, float alpha, int mode, hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && top > 0 && E > 0 && F > 0 && D > 0 && ldh >= D, "pico_moe_experts_plain: bad sizes");
-  PICO_REQUIRE(mode == MOE_MODE_CLIPPED || mode == MOE_MODE_SOFTMAX_SWIGLU, "pico_moe_experts_plain: unknown mode %d", mode);
+  PICO_REQUIRE(mode >= MOE_MODE_CLIPPED && mode <= MOE_MODE_CLIPPED_OUT, "pico_moe_experts_plain: unknown mode %d", mode);
   if (T == 0) return 0;
   const dim3 g1(T * top, (F + 15) / 16), g2(T, (D + 15) / 16);
   PICO_REQUIRE(g1.y <= 65535 && g2.y <= 65535, "pico_moe_experts_plain: sizes beyond the grid");
@@ -413,6 +417,141 @@ extern "C" int pico_moe_router_top_softmax(const void* x, int ldx, int dtype, co
 #undef LAUNCH
   PICO_REQUIRE(E <= 8192, "pico_moe_router_top_softmax: at most 8192 experts");
   moe_route_top_softmax_kernel<<<(T + 3) / 4, 256, (size_t)4 * E * sizeof(float), stream>>>(z, bias, T, E, rows, top, experts, weights);
+  PICO_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------
+// A fourth way of choosing: scores s = sigmoid(z); the experts form `groups` equal groups of neighbours, a group's score is
+// the sum of its two largest s, and only the experts of the `keep` groups with the largest scores can be chosen: the `top`
+// of them with the largest z, their weights their s as they are.  Among equals the lowest index wins.
+// One workgroup a token; its first wave chooses, out of LDS.
+// ---------------------------------------------------------------------------
+#define ROUTE_MAX_E 2048
+#define ROUTE_FUSED_TOKENS 64      // up to this many tokens one launch makes logits and choice
+
+// zs [E], gs [groups] in LDS (zs filled, behind a barrier); called by every thread of the workgroup.
+__device__ __forceinline__ void route_groups(float* zs, float* gs, int E, int groups, int keep, int top, int* __restrict__ experts,
+                                             float* __restrict__ weights) {
+  const int lane = threadIdx.x & 63, n = E / groups;
+  const bool chooser = threadIdx.x < 64;
+  if (chooser && keep < groups) {
+    for (int g = lane; g < groups; g += 64) {
+      float s1 = -INFINITY, s2 = -INFINITY;            // the two largest of the group
+      for (int i = 0; i < n; i++) {
+        const float z = zs[g * n + i];
+        if (z > s1) { s2 = s1; s1 = z; }
+        else if (z > s2) s2 = z;
+      }
+      gs[g] = 1.0f / (1.0f + expf(-s1)) + (n > 1 ? 1.0f / (1.0f + expf(-s2)) : 0.f);
+    }
+  }
+  __syncthreads();
+  if (chooser && keep < groups) {
+    for (int k = 0; k < keep; k++) {
+      float mx = -INFINITY;
+      int mi = 0x7fffffff;
+      for (int g = lane; g < groups; g += 64) {        // a lane's own entries: it alone reads and writes them here
+        const float v = gs[g];
+        if (v > mx || mi == 0x7fffffff) { mx = v; mi = g; }
+      }
+      wave_first_max(mx, mi);
+      mi = min(mi, groups - 1);
+      if ((mi & 63) == lane) gs[mi] = -INFINITY;       // kept (a score is never that)
+    }
+  }
+  __syncthreads();
+  if (!chooser) return;
+  if (keep < groups)
+    for (int e = lane; e < E; e += 64)
+      if (gs[e / n] != -INFINITY) zs[e] = -INFINITY;   // of a group that is not kept
+  float wk = 0.f;                                      // lane k keeps the k-th chosen expert and its weight
+  int ek = 0;
+  for (int k = 0; k < top; k++) {
+    float mx = -INFINITY;
+    int mi = 0x7fffffff;
+    for (int e = lane; e < E; e += 64) {
+      const float v = zs[e];
+      if (v > mx || mi == 0x7fffffff) { mx = v; mi = e; }
+    }
+    wave_first_max(mx, mi);
+    mi = min(mi, E - 1);
+    if (lane == k) { wk = 1.0f / (1.0f + expf(-mx)); ek = mi; }
+    if ((mi & 63) == lane) zs[mi] = -INFINITY;         // taken
+  }
+  if (lane < top) {
+    experts[lane] = ek;
+    weights[lane] = wk;
+  }
+}
+
+__global__ __launch_bounds__(64) void moe_route_groups_kernel(const float* __restrict__ logits, int E, int groups, int keep, int top,
+                                                              int* __restrict__ experts, float* __restrict__ weights) {
+  __shared__ float zs[ROUTE_MAX_E], gs[ROUTE_MAX_E];
+  const size_t t = blockIdx.x;
+  for (int e = threadIdx.x; e < E; e += 64) zs[e] = logits[t * E + e];
+  __syncthreads();
+  route_groups(zs, gs, E, groups, keep, top, experts + t * top, weights + t * top);
+}
+
+// Few tokens: a workgroup makes its token's logits too, a wave an expert at a time, every sum in the order of
+// moe_logits_kernel.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(1024) void moe_router_groups_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ Wr, int E,
+                                                                 int D, int groups, int keep, int top,
+                                                                 int* __restrict__ experts, float* __restrict__ weights) {
+  __shared__ float zs[ROUTE_MAX_E], gs[ROUTE_MAX_E];
+  const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  const size_t t = blockIdx.x;
+  const T* xr = x + t * ldx;
+  for (int e = threadIdx.x >> 6; e < E; e += nw) {
+    const float* w = Wr + (size_t)e * D;
+    float acc = 0.f;
+    if (VEC) {
+#pragma unroll 4
+      for (int k = lane * 4; k < D; k += 256) {
+        float wv[4], xv[4];
+        load4_f32<float>(w + k, wv);
+        load4_f32<T>(xr + k, xv);
+#pragma unroll
+        for (int j = 0; j < 4; j++) acc = fmaf(xv[j], wv[j], acc);
+      }
+    } else {
+      for (int k = lane; k < D; k += 64) acc = fmaf(load_f32(xr + k), w[k], acc);
+    }
+    acc = wave_sum(acc);
+    if (lane == 0) zs[e] = acc;
+  }
+  __syncthreads();
+  route_groups(zs, gs, E, groups, keep, top, experts + t * top, weights + t * top);
+}
+
+// z [T, E]: room for the logits (used with many tokens only)
+extern "C" int pico_moe_router_groups(const void* x, int ldx, int dtype, const float* Wr, int T, int E, int D, int groups, int keep,
+                                      int top, float* z, int* experts, float* weights, hipStream_t stream) {
+  PICO_REQUIRE(T >= 0 && E > 0 && E <= ROUTE_MAX_E && D > 0 && ldx >= D, "pico_moe_router_groups: bad sizes (at most %d experts)", ROUTE_MAX_E);
+  PICO_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups, "pico_moe_router_groups: %d of %d groups of %d experts", keep, groups, E);
+  PICO_REQUIRE(top >= 1 && top <= MOE_MAX_TOP && top <= keep * (E / groups),
+               "pico_moe_router_groups: %d experts per token of %d that may be chosen (at most %d)", top, keep * (E / groups), MOE_MAX_TOP);
+  PICO_REQUIRE(dtype == PICO_DTYPE_F32 || dtype == PICO_DTYPE_BF16, "pico_moe_router_groups: unknown dtype %d", dtype);
+  if (T == 0) return 0;
+  const size_t esz = dtype == PICO_DTYPE_F32 ? 4 : 2;
+  const bool vec = D % 4 == 0 && ldx % 4 == 0 && (uintptr_t)x % (4 * esz) == 0 && (uintptr_t)Wr % 16 == 0;
+  if (T <= ROUTE_FUSED_TOKENS) {
+    const int threads = 64 * min(16, E);
+#define LAUNCH(TT, V) moe_router_groups_kernel<TT, V><<<T, threads, 0, stream>>>((const TT*)x, ldx, Wr, E, D, groups, keep, top, experts, weights)
+    if (dtype == PICO_DTYPE_F32) { if (vec) LAUNCH(float, true); else LAUNCH(float, false); }
+    else { if (vec) LAUNCH(bf16_t, true); else LAUNCH(bf16_t, false); }
+#undef LAUNCH
+  } else {
+    const dim3 grid((T + ROUTER_TOKENS - 1) / ROUTER_TOKENS, (E + 3) / 4);
+    PICO_REQUIRE(z != nullptr, "pico_moe_router_groups: no room for the logits");
+#define LAUNCH(TT, V) moe_logits_kernel<TT, V><<<grid, 256, 0, stream>>>((const TT*)x, ldx, Wr, T, E, D, z)
+    if (dtype == PICO_DTYPE_F32) { if (vec) LAUNCH(float, true); else LAUNCH(float, false); }
+    else { if (vec) LAUNCH(bf16_t, true); else LAUNCH(bf16_t, false); }
+#undef LAUNCH
+    moe_route_groups_kernel<<<T, 64, 0, stream>>>(z, E, groups, keep, top, experts, weights);
+  }
   PICO_LAUNCH_CHECK();
   return 0;
 }

@@ -21,12 +21,12 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 #define MOE_LD 72          // LDS row stride in bfloat16: 144 bytes, a multiple of 16 that spreads rows over the banks
 
 // mode 0: the clipped activation, the row's weight w already in the input; mode 1: w silu(g) u (the weight on the
-// expert's output, taken in front of the linear second product)
+// expert's output, taken in front of the linear second product); mode 2: w times the clipped activation
 __device__ __forceinline__ float moe_act(float g, float u, float limit, float alpha, int mode, float w) {
   if (mode == 1) return w * (g / (1.0f + expf(-g))) * u;
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+  return (mode == 2 ? w : 1.0f) * (g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
 }
 
 __device__ __forceinline__ void unpack8(const uint4& v, float* f) {
@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void moe_up_rows_kernel(const bf16_t* __restri
   const int e = experts[r];
   if (e < 0 || e >= E || f >= F) return;
   const float wr = weights[r];
-  const float w = mode == 1 ? 1.f : wr;
+  const float w = mode != 0 ? 1.f : wr;
   const bf16_t* x = h + (size_t)(r / top) * ldh;
   const bf16_t* wg = gate_up + ((size_t)e * 2 * F + f) * D;
   const bf16_t* wu = wg + (size_t)F * D;
@@ -92,7 +92,7 @@ __global__ __launch_bounds__(256) void moe_up_rows_kernel(const bf16_t* __restri
 #pragma unroll 2
   for (int k = sub * 8; k < D; k += 128) {
     const uint4 x8 = *reinterpret_cast<const uint4*>(x + k);
-    const uint4 xv = mode == 1 ? x8 : scale8(x8, w);
+    const uint4 xv = mode != 0 ? x8 : scale8(x8, w);
     const uint4 gv = *reinterpret_cast<const uint4*>(wg + k);
     const uint4 uv = *reinterpret_cast<const uint4*>(wu + k);
     float xf[8];
@@ -137,7 +137,7 @@ extern "C" int pico_moe_experts_rows(const void* h, int ldh, const void* gate_up
                                      const float* weights, void* y, float* out, int T, int top, int E, int F, int D,
                                      float limit, float alpha, int mode, hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && top > 0 && E > 0 && F > 0 && D > 0 && ldh >= D, "pico_moe_experts_rows: bad sizes");
-  PICO_REQUIRE(mode == 0 || mode == 1, "pico_moe_experts_rows: unknown mode %d", mode);
+  PICO_REQUIRE(mode >= 0 && mode <= 2, "pico_moe_experts_rows: unknown mode %d", mode);
   PICO_REQUIRE(F % 8 == 0 && D % 8 == 0 && ldh % 8 == 0, "pico_moe_experts_rows: sizes must be multiples of 8");
   PICO_REQUIRE(((uintptr_t)h | (uintptr_t)gate_up | (uintptr_t)down | (uintptr_t)y) % 16 == 0,
                "pico_moe_experts_rows: operands must start on 16 bytes");
@@ -253,7 +253,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const bf16_t* __restri
       const int r = sorted[(size_t)tile * MOE_BM + m];                                    \
       A_OK = r >= 0;                                                                      \
       A_SRC = A + (size_t)(A_OK ? r / top : 0) * lda + sk;                                \
-      A_W = A_OK ? (mode == 1 ? 1.f : weights[r]) : 0.f;                                  \
+      A_W = A_OK ? (mode != 0 ? 1.f : weights[r]) : 0.f;                                  \
       const int f = c0 + (m & 63);                                                        \
       B_OK = f < F;                                                                       \
       B_SRC = W + ((size_t)e * erows + (B_OK ? (m >> 6) * F + f : 0)) * K + sk;           \
@@ -301,7 +301,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const bf16_t* __restri
       bf16_t* as = As + srow * MOE_LD + sk;
       bf16_t* bs = Bs + srow * MOE_LD + sk;
       const bool k_in = k0 + sk < K;
-      const bool scaled = UP && mode != 1;        // mode 1 puts the weight on the activation instead
+      const bool scaled = UP && mode == 0;        // the other modes put the weight on the activation instead
       *reinterpret_cast<uint4*>(as) = keep8(scaled ? scale8(ra0, a_w0) : ra0, a_ok0 && k_in);
       *reinterpret_cast<uint4*>(as + 32 * MOE_LD) = keep8(scaled ? scale8(ra1, a_w1) : ra1, a_ok1 && k_in);
       *reinterpret_cast<uint4*>(as + 64 * MOE_LD) = keep8(scaled ? scale8(ra2, a_w2) : ra2, a_ok2 && k_in);
@@ -332,7 +332,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const bf16_t* __restri
     const int m = wm * 64 + 32 * (i) + 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3);                                     \
     if (UP) {                                                                                                        \
       const int f = c0 + wn * 32 + (lane & 31);                                                                      \
-      const float wrow = (mode == 1 && rows[m] >= 0) ? weights[rows[m]] : 0.f;                                       \
+      const float wrow = (mode != 0 && rows[m] >= 0) ? weights[rows[m]] : 0.f;                                       \
       if (f < F) y[((size_t)tile * MOE_BM + m) * F + f] = f32_to_bf16(moe_act(ACC0[r], ACC1[r], limit, alpha, mode, wrow)); \
     } else {                                                                                                         \
       const int row = rows[m];                                                                                       \
@@ -354,7 +354,7 @@ extern "C" int pico_moe_experts_grouped(const void* h, int ldh, const void* gate
                                         const float* weights, int* sorted, int* tile_expert, int tiles_cap, void* y,
                                         float* out, int T, int top, int E, int F, int D, float limit, float alpha,
                                         int mode, hipStream_t stream) {
-  PICO_REQUIRE(mode == 0 || mode == 1, "pico_moe_experts_grouped: unknown mode %d", mode);
+  PICO_REQUIRE(mode >= 0 && mode <= 2, "pico_moe_experts_grouped: unknown mode %d", mode);
   PICO_REQUIRE(T >= 0 && top > 0 && E > 0 && F > 0 && D > 0 && ldh >= D, "pico_moe_experts_grouped: bad sizes");
   PICO_REQUIRE(E <= MOE_SORT_MAX_E, "pico_moe_experts_grouped: at most %d experts", MOE_SORT_MAX_E);
   PICO_REQUIRE(F % 8 == 0 && D % 8 == 0 && ldh % 8 == 0, "pico_moe_experts_grouped: sizes must be multiples of 8");

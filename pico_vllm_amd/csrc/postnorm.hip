@@ -3,8 +3,8 @@
 //   pico_norm_add:        x[t] += rms(y[t]) * w                          (y: the sublayer's output)
 //                         or, with two outputs a and b and a weight each,
 //                         x[t] += rms( (rms(a[t]) * wa + rms(b[t]) * wb) / 2 ) * w
-//   pico_norm_add_norm:   x[t] += rms(y[t]) * w, and out[t] = rms(x[t]) * w_next (the next sublayer's norm in front of it) or,
-//                         without w_next, x[t] itself in the activations' storage type
+//   pico_norm_add_norm:   x[t] += rms(y[t]) * w (+ a vector, the same for every row), and out[t] = rms(x[t]) * w_next (the next
+//                         sublayer's norm in front of it) or, without w_next, x[t] itself in the activations' storage type
 //   pico_stream_rmsnorm:  x[t] <- rms(x[t]) * w
 //   rms(v) = v / sqrt(mean(v^2) + eps).  Both can leave a copy of the new x in the activations' storage type, which is
 //   what the next sublayer reads.
@@ -101,7 +101,7 @@ template <typename TY, typename TO, int V, int VPT>
 __global__ __launch_bounds__(1024) void norm_add_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, int slabs,
                                                              size_t slab_stride, const float* __restrict__ w, float eps,
                                                              const float* __restrict__ w_next, float eps_next, TO* __restrict__ out,
-                                                             int ld_out, int H) {
+                                                             int ld_out, int H, const float* __restrict__ vec) {
   __shared__ float scratch[16];
   const size_t base = (size_t)blockIdx.x * H;
   float yv[VPT][V], xv[VPT][V], wv[VPT][V];
@@ -124,6 +124,11 @@ __global__ __launch_bounds__(1024) void norm_add_norm_kernel(float* __restrict__
 #pragma unroll
       for (int k = 0; k < V; k++) yv[j][k] += more[j][k];
   }
+  float add[VPT][V];
+  if (vec) {
+#pragma unroll
+    for (int j = 0; j < VPT; j++) load_v<float, V>(vec + (ok[j] ? (j * (int)blockDim.x + (int)threadIdx.x) * V : 0), add[j]);
+  }
   float ss = 0.f;
 #pragma unroll
   for (int j = 0; j < VPT; j++)
@@ -136,6 +141,7 @@ __global__ __launch_bounds__(1024) void norm_add_norm_kernel(float* __restrict__
 #pragma unroll
     for (int k = 0; k < V; k++) {
       xv[j][k] += yv[j][k] * r * wv[j][k];
+      if (vec) xv[j][k] += add[j][k];
       ss = ok[j] ? fmaf(xv[j][k], xv[j][k], ss) : ss;
     }
     if (ok[j]) store_v<float, V>(x + base + (j * (int)blockDim.x + (int)threadIdx.x) * V, xv[j]);
@@ -220,13 +226,13 @@ extern "C" int pico_norm_add(float* x, const void* a, int a_dtype, int a_slabs, 
 
 extern "C" int pico_norm_add_norm(float* x, const void* y, int y_dtype, int slabs, long long slab_stride, const float* w, float eps,
                                   const float* w_next, float eps_next, void* out, int out_dtype, int ld_out, int T, int H,
-                                  hipStream_t stream) {
+                                  const float* vec, hipStream_t stream) {
   PICO_REQUIRE(T >= 0 && H > 0 && H <= POSTNORM_MAX_H, "pico_norm_add_norm: a width of 1 to %d, got %d", POSTNORM_MAX_H, H);
   PICO_REQUIRE(x && y && w && slabs >= 1 && (slabs == 1 || y_dtype == PICO_DTYPE_F32), "pico_norm_add_norm: bad operands (partial sums are float32)");
   PICO_REQUIRE(eps > 0.f && (w_next == nullptr || (eps_next > 0.f && out)) && (out == nullptr || ld_out >= H), "pico_norm_add_norm: bad operands");
   PICO_REQUIRE((y_dtype | 1) == 1 && (out_dtype | 1) == 1, "pico_norm_add_norm: unknown dtype");
   if (T == 0) return 0;
-  const uintptr_t all = (uintptr_t)x | (uintptr_t)y | (uintptr_t)w | (uintptr_t)w_next | (uintptr_t)out;
+  const uintptr_t all = (uintptr_t)x | (uintptr_t)y | (uintptr_t)w | (uintptr_t)w_next | (uintptr_t)out | (uintptr_t)vec;
   // (every pointer on 16 bytes and rows of whole fours: then so is every row, or on 8 bytes where storage is bfloat16)
   const bool four = H % 4 == 0 && all % 16 == 0 && (out == nullptr || ld_out % 4 == 0) && (slabs == 1 || slab_stride % 4 == 0);
   const int units = four ? H / 4 : H;
@@ -234,7 +240,7 @@ extern "C" int pico_norm_add_norm(float* x, const void* y, int y_dtype, int slab
   const int threads = ((units + vpt - 1) / vpt + 63) / 64 * 64;
 #define LAUNCH(TY, TO, V, VPT)                                                                                                   \
   norm_add_norm_kernel<TY, TO, V, VPT><<<T, threads, 0, stream>>>(x, (const TY*)y, slabs, (size_t)slab_stride, w, eps, w_next,   \
-                                                                  eps_next, (TO*)out, ld_out, H)
+                                                                  eps_next, (TO*)out, ld_out, H, vec)
 #define PICK(TY, TO)                              \
   do {                                            \
     if (four && vpt == 1) LAUNCH(TY, TO, 4, 1);   \

@@ -15,7 +15,6 @@
 
 #define SSM_MAX_TAPS 16
 
-__device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
 // what follows the convolution: silu, or nothing
 __device__ __forceinline__ float conv_act(float v, int silu) { return silu ? silu_f(v) : v; }
 // the decay exp(dt A) of an element: the library's exponential in the 32-bit engine; with bfloat16 storage the

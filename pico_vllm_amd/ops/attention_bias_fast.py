@@ -25,13 +25,15 @@ class FastBiasAttention:
     def __init__(self, nq: int, nkv: int, key_dim: int, value_dim: int, scale: float, window: int = 0,
                  temp_coef: float = 0.0, temp_every: int = 0, slope_span: float = 0.0, softcap: float = 0.0,
                  keep_first: int = 0, gated: bool = False, chunk: int = 0, sink: bool = False, gate_heads: bool = False,
-                 v_div: int = 1, out_f32: bool = False):
+                 v_div: int = 1, out_f32: bool = False, out_scale: float = 1.0):
         self.nq, self.nkv, self.dk, self.dv = nq, nkv, key_dim, value_dim
         self.scale, self.window, self.temp_coef, self.temp_every, self.slope_span = scale, window, temp_coef, temp_every, slope_span
         self.softcap, self.keep_first, self.gated = float(softcap), int(keep_first), bool(gated)
         # chunked visibility instead of a window, a sink in the softmax, a gate of one number a head, several kv heads
         # over one head of values, float32 output (see csrc/attention_bias.hip)
         self.chunk, self.sink, self.gate_heads, self.v_div, self.out_f32 = int(chunk), bool(sink), bool(gate_heads), int(v_div), bool(out_f32)
+        self.sinks: Optional[torch.Tensor] = None        # the sinks' scores, float32 [nq] (none: 0)
+        self.out_scale = float(out_scale)                # on the output
         self.lib = library.attention_bias_library(key_dim, value_dim)
         if self.lib.pico_attnb_key_dim() != key_dim or self.lib.pico_attnb_value_dim() != value_dim:
             raise KernelError("attention library was built for other sizes")
@@ -42,7 +44,7 @@ class FastBiasAttention:
         # (that kernel knows no cap on the scores, no kept first positions and no gate)
         if key_dim == value_dim and key_dim % 32 == 0 and attention_fast.supported(nq, nkv, key_dim, window) \
                 and not (self.softcap > 0 or (self.keep_first > 0 and window > 0) or self.gated or self.chunk or self.sink
-                         or self.v_div != 1 or self.out_f32):
+                         or self.v_div != 1 or self.out_f32 or self.out_scale != 1.0):
             self.tuned = attention_fast.FastAttention(nq, nkv, key_dim, window)
 
     def split(self, num_tokens: int) -> bool:
@@ -104,8 +106,11 @@ class FastBiasAttention:
                                  or gate.stride(1) != 1 or gate.shape[1] < (self.nq if self.gate_heads else self.nq * self.dv)
                                  or (not self.gate_heads and ((T > 1 and gate.stride(0) % 4) or gate.data_ptr() % 8))):
             raise KernelError("the gate must be bfloat16 [T, >= nq*dv] with unit stride along the row and 8-byte aligned rows")
+        odt = torch.float32 if self.out_f32 else torch.bfloat16
         if out is None:
-            out = torch.empty(T, self.nq * self.dv, dtype=torch.float32 if self.out_f32 else torch.bfloat16, device=q.device)
+            out = torch.empty(T, self.nq * self.dv, dtype=odt, device=q.device)
+        elif not out.is_cuda or tuple(out.shape) != (T, self.nq * self.dv) or out.dtype != odt or out.stride(1) != 1:
+            raise KernelError("attention: out has the wrong shape or dtype")
         if split is None:
             split = self.split(T)
         if chunks is None:
@@ -122,12 +127,13 @@ class FastBiasAttention:
             c_float(self.scale), self.window, c_float(self.temp_coef), self.temp_every, c_float(self.slope_span),
             1 if split else 0, chunks, _ptr(parts_o), _ptr(parts_ml), c_float(self.softcap), self.keep_first, _ptr(gate),
             0 if gate is None else (gate.stride(0) if T > 1 else gate.shape[1]), self.chunk, 1 if self.sink else 0,
-            1 if self.gate_heads else 0, self.v_div, 1 if self.out_f32 else 0, _stream()))
+            1 if self.gate_heads else 0, self.v_div, 1 if self.out_f32 else 0, _ptr(self.sinks), c_float(self.out_scale),
+            out.stride(0) if T > 1 else self.nq * self.dv, _stream()))
         return out
 
-    def __call__(self, qkv, cache, block_table, ctx, gate=None):
+    def __call__(self, qkv, cache, block_table, ctx, gate=None, out=None):
         split, chunks, shape = self.plan(ctx)
-        if shape and cache.k.numel() * cache.k.element_size() < (1 << 32):
+        if shape and out is None and cache.k.numel() * cache.k.element_size() < (1 << 32):
             B = ctx.num_seqs
             order, build = None, False
             if B >= 2:      # several sequences: the list of their query tiles, longest first, written by the first layer
@@ -139,15 +145,17 @@ class FastBiasAttention:
                                       teams=shape, order=order, order_build=build,
                                       scored=(self.temp_coef, self.temp_every, self.slope_span))
         return self.run(qkv, cache.k, cache.v, block_table, ctx.cu_seqlens, ctx.positions, ctx.num_seqs,
-                        split=split, chunks=chunks, gate=gate)
+                        split=split, chunks=chunks, gate=gate, out=out)
 
 
 def choose(mixer) -> Optional[FastBiasAttention]:
     """The matrix-core kernel for this mixer's sizes, or None where the plain kernel serves."""
     if not supported(mixer.dk, mixer.dv):
         return None
-    return FastBiasAttention(mixer.nq, mixer.nkv, mixer.dk, mixer.dv, mixer.scale, mixer.window, mixer.temp_coef,
+    fast = FastBiasAttention(mixer.nq, mixer.nkv, mixer.dk, mixer.dv, mixer.scale, mixer.window, mixer.temp_coef,
                              mixer.temp_every, mixer.slope_span, getattr(mixer, "softcap", 0.0),
                              getattr(mixer, "keep_first", 0), getattr(mixer, "gated", False), getattr(mixer, "chunk", 0),
                              getattr(mixer, "sink", False), getattr(mixer, "gate_heads", False), getattr(mixer, "v_div", 1),
-                             getattr(mixer, "out_f32", False))
+                             getattr(mixer, "out_f32", False), getattr(mixer, "out_scale", 1.0))
+    fast.sinks = getattr(mixer, "sinks", None)
+    return fast

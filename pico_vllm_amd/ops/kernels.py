@@ -78,10 +78,12 @@ def _i32(t: torch.Tensor, name: str, n: Optional[int] = None) -> None:
         raise KernelError(f"{name} has {t.numel()} entries, {n} are needed")
 
 
-def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
-    """out[t] = table[ids[t]] * scale as float32 rows (the residual stream)."""
-    _gpu(table, ids)
+def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None, scale: float = 1.0,
+              vector: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[t] = table[ids[t]] * scale (+ ``vector`` [H] float32) as float32 rows (the residual stream)."""
+    _gpu(table, ids, vector)
     V, H = table.shape
+    _vec(vector, H, "the vector added to every row")
     T = ids.numel()
     _i32(ids, "ids")
     if not table.is_contiguous():
@@ -91,7 +93,7 @@ def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor
     elif out.shape != (T, H) or out.dtype != torch.float32 or not out.is_contiguous():
         raise KernelError("embedding: out must be a contiguous float32 [T, H] tensor")
     lib = library.core()
-    _check(lib, lib.pico_embedding(_ptr(table), _dt(table), _ptr(ids), _ptr(out), T, H, V, c_float(scale), _stream()))
+    _check(lib, lib.pico_embedding(_ptr(table), _dt(table), _ptr(ids), _ptr(out), T, H, V, c_float(scale), _ptr(vector), _stream()))
     return out
 
 
@@ -181,6 +183,18 @@ def residual_add(resid: torch.Tensor, delta: torch.Tensor) -> torch.Tensor:
     return resid
 
 
+def add_vector(resid: torch.Tensor, vector: torch.Tensor) -> torch.Tensor:
+    """resid (float32 [T, H], in place) += ``vector`` [H] float32, in every row."""
+    _gpu(resid, vector)
+    T, H = resid.shape
+    if resid.dtype != torch.float32 or not resid.is_contiguous():
+        raise KernelError("the residual stream must be contiguous float32")
+    _vec(vector, H, "the vector added to every row")
+    lib = library.core()
+    _check(lib, lib.pico_add_vector(_ptr(resid), _ptr(vector), T, H, _stream()))
+    return resid
+
+
 def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     _gpu(gate_up)
     T, I2 = gate_up.shape
@@ -256,7 +270,7 @@ def gemm_bf16(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = N
     return out
 
 
-EPI_BF16, EPI_F32, EPI_SWIGLU, EPI_RELU2, EPI_F32_ADD, EPI_CLIPPED, EPI_GELU_TOKEN = 0, 1, 2, 3, 4, 5, 6
+EPI_BF16, EPI_F32, EPI_SWIGLU, EPI_RELU2, EPI_F32_ADD, EPI_CLIPPED, EPI_GELU_TOKEN, EPI_GELU = 0, 1, 2, 3, 4, 5, 6, 7
 MAX_HEAD_DIM = 256          # the largest head size any attention kernel takes
 
 
@@ -291,7 +305,8 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
     -> bf16 [M, N / 2] = silu(gate) * up; EPI_RELU2 -> bf16 [M, N] = max(x w^T + bias, 0)^2; EPI_F32_ADD: ``out``
     (contiguous float32 [M, N], a residual stream) += x w^T + bias, every element by one writer; EPI_CLIPPED (w = [gate;
     up], ``clip`` = (limit, alpha)) -> bf16 [M, N / 2] as ``clipped_glu``; EPI_GELU_TOKEN (``token_rows`` = (ids int32 [M],
-    table bf16 [rows, columns], first column)) -> bf16 [M, N] as ``gelu_token``."""
+    table bf16 [rows, columns], first column)) -> bf16 [M, N] as ``gelu_token``; EPI_GELU -> bf16 [M, N] = gelu(x w^T + bias)
+    with the error function."""
     _gpu(a, w, bias)
     M, K = a.shape
     N, K2 = w.shape
@@ -627,18 +642,27 @@ def add_rows(resid: torch.Tensor, table: torch.Tensor, idx: torch.Tensor) -> tor
     return resid
 
 
-def relu2(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """max(x, 0)^2 element by element (``out=x``: in place)."""
+def _activation(entry: str, x: torch.Tensor, out: Optional[torch.Tensor]) -> torch.Tensor:
     _gpu(x, out)
     if not x.is_contiguous():
-        raise KernelError("relu2: the input must be contiguous")
+        raise KernelError(f"{entry}: the input must be contiguous")
     if out is None:
         out = torch.empty_like(x)
     elif out.shape != x.shape or out.dtype != x.dtype or not out.is_contiguous():
-        raise KernelError("relu2: out has the wrong shape or dtype")
+        raise KernelError(f"{entry}: out has the wrong shape or dtype")
     lib = library.core()
-    _check(lib, lib.pico_relu2(_ptr(x), _ptr(out), _dt(x), c_ll(x.numel()), _stream()))
+    _check(lib, getattr(lib, entry)(_ptr(x), _ptr(out), _dt(x), c_ll(x.numel()), _stream()))
     return out
+
+
+def relu2(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """max(x, 0)^2 element by element (``out=x``: in place)."""
+    return _activation("pico_relu2", x, out)
+
+
+def gelu(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x / 2 (1 + erf(x / sqrt 2)) element by element (``out=x``: in place)."""
+    return _activation("pico_gelu", x, out)
 
 
 def _check_cache2(k_cache: torch.Tensor, v_cache: torch.Tensor, nkv: int, dk: int, dv: int, nv: Optional[int] = None):
@@ -682,15 +706,18 @@ def attn_bias_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     window: int = 0, temp_coef: float = 0.0, temp_every: int = 0, slope_span: float = 0.0,
                     out: Optional[torch.Tensor] = None, softcap: float = 0.0, keep_first: int = 0,
                     gate: Optional[torch.Tensor] = None, chunk: int = 0, sink: bool = False, gate_heads: bool = False,
-                    v_div: int = 1, out_f32: bool = False) -> torch.Tensor:
+                    v_div: int = 1, out_f32: bool = False, sinks: Optional[torch.Tensor] = None,
+                    out_scale: float = 1.0) -> torch.Tensor:
     """Attention with a distance penalty slope_h (i - j), slope_h = 2^(-slope_span (h + 1) / nq), and the query
     temperature 1 + temp_coef ln(floor((i + 1) / temp_every) + 1) on the scores.  q: [T, >= nq * dk]; returns [T, nq * dv].
     ``softcap`` > 0: scores <- softcap tanh(scores / softcap).  ``keep_first``: with a window, keys at positions below it
     stay visible.  ``gate`` [T, >= nq * dv] (row stride free): the output is multiplied with sigmoid(gate); with
     ``gate_heads`` the gate is [T, >= nq], one number a head.  ``chunk`` > 0 (instead of a window): key j <= i is seen iff
-    floor(i / chunk) == floor(j / chunk).  ``sink``: the softmax's denominator gains a 1.  ``v_div``: kv head g reads value
-    head g // v_div (the value pages hold nkv // v_div heads).  ``out_f32``: the output is float32 whatever q's dtype."""
-    _gpu(q, k_cache, v_cache, block_table, positions, token_seq, gate)
+    floor(i / chunk) == floor(j / chunk).  ``sink``: the softmax's denominator gains a 1, or exp(``sinks``[h]) (float32 [nq]).
+    ``v_div``: kv head g reads value head g // v_div (the value pages hold nkv // v_div heads).  ``out_f32``: the output is
+    float32 whatever q's dtype.  ``out_scale``: a factor on the output.  ``out``: its rows may be strided."""
+    _gpu(q, k_cache, v_cache, block_table, positions, token_seq, gate, out, sinks)
+    _vec(sinks, nq, "the sinks' scores")
     T = q.shape[0]
     if q.dim() != 2 or q.stride(1) != 1 or q.shape[1] < nq * dk:
         raise KernelError("q must be [T, >= nq*dk] with unit stride along the row")
@@ -706,7 +733,7 @@ def attn_bias_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     odt = torch.float32 if out_f32 else q.dtype
     if out is None:
         out = torch.empty(T, nq * dv, dtype=odt, device=q.device)
-    elif out.shape != (T, nq * dv) or out.dtype != odt or not out.is_contiguous():
+    elif out.shape != (T, nq * dv) or out.dtype != odt or out.stride(1) != 1:
         raise KernelError("attention: out has the wrong shape or dtype")
     if gate is not None and (gate.dtype != q.dtype or gate.dim() != 2 or gate.stride(1) != 1 or gate.shape[0] != T
                              or gate.shape[1] < (nq if gate_heads else nq * dv)):
@@ -717,7 +744,8 @@ def attn_bias_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                                          T, nq, nkv, dk, dv, P, window, c_float(scale), c_float(temp_coef), temp_every,
                                          c_float(slope_span), pages, c_float(softcap), keep_first, _ptr(gate),
                                          0 if gate is None else (gate.stride(0) if T > 1 else gate.shape[1]), chunk,
-                                         1 if sink else 0, 1 if gate_heads else 0, v_div, 1 if out_f32 else 0, _stream()))
+                                         1 if sink or sinks is not None else 0, 1 if gate_heads else 0, v_div, 1 if out_f32 else 0,
+                                         _ptr(sinks), c_float(out_scale), out.stride(0) if T > 1 else nq * dv, _stream()))
     return out
 
 
@@ -771,13 +799,14 @@ GLA_MAX_KEY_DIM = 256
 def gla_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: Optional[torch.Tensor], cu_seqlens: torch.Tensor,
              state_slots: torch.Tensor, state: torch.Tensor, num_seqs: int, heads: int, dk: int, dv: int,
              qscale: float, chunk: int = 0, decay_from: Optional[tuple] = None,
-             head_decay: Optional[torch.Tensor] = None) -> torch.Tensor:
+             head_decay: Optional[torch.Tensor] = None, silu: bool = False) -> torch.Tensor:
     """The recurrence S <- diag(exp(log_decay_t)) S + k_t v_t^T, o_t = S^T q_t qscale, for every sequence of the step from
     its state slot (``state`` float32 [slots, heads, dk, dv], updated in place).  Returns o float32 [T, heads * dv].
     ``chunk`` > 0: sequences are cut into chunks of that many tokens that run side by side (every chunk from zero, a walk
     over the chunks' states, every chunk again from its true state): the same sums in another order.
     ``log_decay`` None (whole walks only): the decays are made inside the launch from ``decay_from`` = (column of the
-    low-rank activations in x, a2 [heads * dk, R], bias float32 or None, tau), as ``gla_decay`` makes them."""
+    low-rank activations in x, a2 [heads * dk, R], bias float32 or None, tau), as ``gla_decay`` makes them.
+    ``silu``: q, k and v go through z sigmoid(z) as they are read."""
     _gpu(x, log_decay, cu_seqlens, state_slots, state)
     T = x.shape[0]
     if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] < max(q_col + heads * dk, k_col + heads * dk, v_col + heads * dv):
@@ -817,7 +846,7 @@ def gla_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: Opt
     _check(lib, lib.pico_gla_scan(_ptr(x), x.stride(0) if T > 1 else x.shape[1], _dt(x), q_col, k_col, v_col, _ptr(log_decay),
                                   _ptr(cu_seqlens), _ptr(state_slots), _ptr(state), _ptr(out), num_seqs, T, heads, dk, dv,
                                   c_float(qscale), state.shape[0], chunk, max_chunks, _ptr(ws), _ptr(ws_decay), _ptr(a2),
-                                  _ptr(a2_bias), a_col, R, c_float(tau), _ptr(head_decay), _stream()))
+                                  _ptr(a2_bias), a_col, R, c_float(tau), _ptr(head_decay), 1 if silu else 0, _stream()))
     return out
 
 
@@ -837,6 +866,27 @@ def gla_out(o: torch.Tensor, x: torch.Tensor, g_col: int, weight: torch.Tensor, 
     lib = library.core()
     _check(lib, lib.pico_gla_out(_ptr(o), _ptr(x[:, g_col:]), x.stride(0) if T > 1 else x.shape[1], _dt(x), _ptr(weight),
                                  c_float(eps), _ptr(out), T, heads, dv, 1 if sigmoid_gate else 0, _stream()))
+    return out
+
+
+def gated_row_norm(o: torch.Tensor, x: torch.Tensor, g_col: int, weight: torch.Tensor, eps: float,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """[T, N] of x's dtype: the rows of ``o`` (float32 [T, N]) RMS-normed over all N entries with ``weight`` [N], times the
+    sigmoid of the gate (columns g_col .. of x).  ``out``: where to (its rows may be strided)."""
+    _gpu(o, x, weight, out)
+    T, N = o.shape
+    if o.dtype != torch.float32 or not o.is_contiguous():
+        raise KernelError("gated_row_norm: o must be contiguous float32")
+    if x.dim() != 2 or x.shape[0] != T or x.stride(1) != 1 or x.shape[1] < g_col + N:
+        raise KernelError("gated_row_norm: the rows do not hold the gate")
+    _vec(weight, N, "norm weight")
+    if out is None:
+        out = torch.empty(T, N, dtype=x.dtype, device=x.device)
+    elif tuple(out.shape) != (T, N) or out.dtype != x.dtype or out.stride(1) != 1:
+        raise KernelError("gated_row_norm: out has the wrong shape or dtype")
+    lib = library.core()
+    _check(lib, lib.pico_gated_row_norm(_ptr(o), _ptr(x[:, g_col:]), x.stride(0) if T > 1 else x.shape[1], _dt(x), _ptr(weight),
+                                        c_float(eps), _ptr(out), out.stride(0) if T > 1 else N, T, N, _stream()))
     return out
 
 
@@ -904,6 +954,26 @@ def moe_router_softmax(x: torch.Tensor, w_router: torch.Tensor, correction: Opti
     return experts, weights
 
 
+def moe_router_groups(x: torch.Tensor, w_router: torch.Tensor, groups: int, keep: int, top: int):
+    """Router and choice: z = x w_router^T in float32, s = sigmoid(z); of ``groups`` equal groups of neighbouring experts the
+    ``keep`` ones with the largest sums of their two largest s; among their experts the ``top`` largest z (the lowest index
+    among equals).  Returns (experts int32 [T, top], their s float32 [T, top])."""
+    _gpu(x, w_router)
+    T, D = x.shape
+    E = w_router.shape[0]
+    if w_router.dtype != torch.float32 or w_router.dim() != 2 or w_router.shape[1] != D or not w_router.is_contiguous():
+        raise KernelError(f"moe_router_groups: the router matrix must be contiguous float32 [experts, {D}]")
+    if x.stride(1) != 1:
+        raise KernelError("moe_router_groups: activations must have unit stride along the row")
+    z = torch.empty(T, E, dtype=torch.float32, device=x.device)
+    experts = torch.empty(T, top, dtype=torch.int32, device=x.device)
+    weights = torch.empty(T, top, dtype=torch.float32, device=x.device)
+    lib = library.core()
+    _check(lib, lib.pico_moe_router_groups(_ptr(x), x.stride(0) if T > 1 else D, _dt(x), _ptr(w_router), T, E, D, groups, keep, top,
+                                           _ptr(z), _ptr(experts), _ptr(weights), _stream()))
+    return experts, weights
+
+
 def moe_identity(h: torch.Tensor, experts: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, num_experts: int) -> torch.Tensor:
     """Experts numbered from ``num_experts`` on hand their input on: ``out`` float32 [T, D] += sum of their weights
     times h; or, for a stack [top, T, D] of slabs (one a slot), the slab rows of such slots = weight times h (no
@@ -923,7 +993,8 @@ def moe_identity(h: torch.Tensor, experts: torch.Tensor, weights: torch.Tensor, 
     return out
 
 
-MOE_CLIPPED, MOE_SWIGLU = 0, 1      # the experts' activation: clipped with the weight on the input; silu(g) u, weight on the output
+# the experts' activation: clipped with the weight on the input; silu(g) u, weight on the output; clipped, weight on the output
+MOE_CLIPPED, MOE_SWIGLU, MOE_CLIPPED_OUT = 0, 1, 2
 
 
 def _check_experts(h, gate_up, down, experts, weights, who):
@@ -1300,12 +1371,13 @@ def norm_add(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: fl
 
 
 def norm_add_norm(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,
-                  next_eps: float = 0.0, out: Optional[torch.Tensor] = None,
-                  out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
-    """resid (float32 [T, H], in place) += rms(y) * weight; y: [T, H], or a float32 stack [S, T, H] whose slabs are added up
+                  next_eps: float = 0.0, out: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None,
+                  vector: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """resid (float32 [T, H], in place) += rms(y) * weight (+ ``vector`` [H] float32, in every row); y: [T, H], or a float32 stack [S, T, H] whose slabs are added up
     first.  The same launch leaves rows beside the stream, in ``out`` ([T, H], row stride free) or a tensor made here of
     ``out_dtype``: the new stream itself or, with ``next_weight``, its RMS norm with that weight.  Neither given: nothing."""
-    _gpu(resid, y, weight, next_weight, out)
+    _gpu(resid, y, weight, next_weight, out, vector)
+    _vec(vector, resid.shape[1], "the vector added to every row")
     T, H = resid.shape
     if resid.dtype != torch.float32 or not resid.is_contiguous():
         raise KernelError("the residual stream must be contiguous float32")
@@ -1320,7 +1392,7 @@ def norm_add_norm(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, ep
     lib = library.core()
     _check(lib, lib.pico_norm_add_norm(_ptr(resid), _ptr(y), _dt(y), slabs, c_ll(T * H), _ptr(weight), c_float(eps), _ptr(next_weight),
                                        c_float(next_eps), _ptr(out), _dt(out) if out is not None else F32,
-                                       out.stride(0) if out is not None and T > 1 else H, T, H, _stream()))
+                                       out.stride(0) if out is not None and T > 1 else H, T, H, _ptr(vector), _stream()))
     return out
 
 
@@ -1369,10 +1441,12 @@ QK_NORM_NONE, QK_NORM_UNIT, QK_NORM_ROW = 0, 1, 2
 def qk_norm_store(x: torch.Tensor, q_col: int, k_col: int, v_col: int, nq: int, nk: int, nv: int, dk: int, dv: int, maps: int,
                   norm_mode: int, wq: Optional[torch.Tensor], wk: Optional[torch.Tensor], eps: float,
                   cos_sin: Optional[torch.Tensor], rotary_dim: int, slots: Optional[torch.Tensor],
-                  k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor]) -> torch.Tensor:
+                  k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], pairs: bool = False) -> torch.Tensor:
     """RMS norm of the nq query and nk key units of dk entries in every row of x (QK_NORM_UNIT: every unit by itself,
     weights [dk]; QK_NORM_ROW: all units of a row at once, weights [nq * dk] and [nk * dk]), then the first ``rotary_dim``
-    entries of every unit turned (entry i with i + rotary_dim / 2; ``cos_sin`` from ``rope_table``).  Returns the queries
+    entries of every unit turned (entry i with i + rotary_dim / 2, or with ``pairs`` entry 2 i with 2 i + 1; ``cos_sin`` from
+    ``rope_table``).  QK_NORM_UNIT may come without weights (a rotation keeps a unit's length, so that norm may as well stand
+    behind it).  Returns the queries
     [T, nq * dk]; with ``maps`` > 1 (a head holds that many units) in the order (kv group, map, head in group).  Keys go
     to ``k_cache`` [pages, nk, P, dk] and columns v_col .. of x, as they are, to ``v_cache`` [pages, nv, dv, P] at
     ``slots`` (negative: nothing); without a cache only the queries are made."""
@@ -1387,7 +1461,7 @@ def qk_norm_store(x: torch.Tensor, q_col: int, k_col: int, v_col: int, nq: int, 
     if norm_mode != QK_NORM_NONE:
         n = dk if norm_mode == QK_NORM_UNIT else None
         _vec(wq, n or nq * dk, "the queries' norm weight"); _vec(wk, n or nk * dk, "the keys' norm weight")
-        if wq is None or wk is None:
+        if (wq is None) != (wk is None) or (wq is None and norm_mode == QK_NORM_ROW):
             raise KernelError("qk_norm_store: a norm needs its weights")
     if rotary_dim % 2 or not 0 <= rotary_dim <= dk:
         raise KernelError(f"qk_norm_store: {rotary_dim} turned entries do not fit a unit of {dk}")
@@ -1403,7 +1477,7 @@ def qk_norm_store(x: torch.Tensor, q_col: int, k_col: int, v_col: int, nq: int, 
     _check(lib, lib.pico_qk_norm_store(_ptr(x), _dt(x), x.stride(0) if T > 1 else x.shape[1], q_col, k_col, v_col, nq, nk, nv, dk,
                                        dv, maps, norm_mode, _ptr(wq), _ptr(wk), c_float(eps),
                                        _ptr(cos_sin) if rotary_dim else None, rotary_dim, _ptr(slots), _ptr(q_out), _ptr(k_cache),
-                                       _ptr(v_cache), T, P, pages, _stream()))
+                                       _ptr(v_cache), T, P, pages, 1 if pairs else 0, _stream()))
     return q_out
 
 

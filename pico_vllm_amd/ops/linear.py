@@ -153,6 +153,13 @@ class Linear:
         y = self(x)
         return kernels.relu2(y, out=y)
 
+    def gelu(self, x: torch.Tensor) -> torch.Tensor:
+        """gelu(x W^T + b) with the error function; with few rows the epilogue of the weight-streaming kernel."""
+        if self.weight.dtype == torch.bfloat16 and kernels.skinny_ok(x, self.weight):
+            return kernels.gemm_skinny(x, self.weight, self.bias_f32, kernels.EPI_GELU)
+        y = self(x)
+        return kernels.gelu(y, out=y)
+
     def add_into(self, x: torch.Tensor, resid: torch.Tensor) -> torch.Tensor:
         """resid (float32 [T, N], in place) += x W^T + b.  With few rows the sum is the epilogue of the weight-streaming
         kernel; otherwise the product and then the sum."""
@@ -173,11 +180,11 @@ class Linear:
         return self(x, out_dtype=torch.float32).unsqueeze(0)
 
     def partial(self, x: torch.Tensor) -> torch.Tensor:
-        """x W^T as something a norm's ``add_norm`` takes as delta: [T, N], or, when the matrix is
+        """x W^T + b as something a norm's ``add_norm`` takes as delta: [T, N], or, when the matrix is
         too small to fill the chip with one workgroup per output tile, a float32 stack [S, T, N] of
-        partial sums over S ranges of k, which the norm kernel adds up."""
-        if self.weight.dtype == torch.bfloat16 and self.bias is None and kernels.skinny_ok(x, self.weight):
+        partial sums over S ranges of k (the bias in the first), which the norm kernel adds up."""
+        if self.weight.dtype == torch.bfloat16 and kernels.skinny_ok(x, self.weight):
             splits = kernels.skinny_k_splits(self.out_features, self.in_features)
             if splits > 1:
-                return kernels.gemm_skinny(x, self.weight, None, kernels.EPI_F32, splits)
+                return kernels.gemm_skinny(x, self.weight, self.bias_f32, kernels.EPI_F32, splits)
         return self(x)

@@ -208,6 +208,56 @@ class Mixer(Part):
         raise NotImplementedError
 
 
+class OpenMixer(Mixer):
+    """A mixer that is one matrix product, a core and one more product, and lets an arrangement of several mixers make the
+    products of all of them together (``parts.pair.MixerSum``).  By itself it makes its own.
+
+    A subclass names the matrices that read the input, in the order of the product's columns (``in_matrices``), and the
+    output's (``out_matrix``), and implements the core: from the product's rows to what the output's product reads."""
+
+    proj = None                      # of the mixer by itself
+    o = None
+
+    def in_matrices(self) -> List[tuple]:
+        """[(tensor name, rows)] in the order of the product's columns."""
+        raise NotImplementedError
+
+    def out_matrix(self) -> tuple:
+        """(tensor name, columns)."""
+        raise NotImplementedError
+
+    def core_params(self) -> List[ParamSpec]:
+        """The tensors beside those matrices."""
+        return []
+
+    def load_core(self, tensors: Dict[str, torch.Tensor], device, dtype, scale: float = 1.0) -> None:
+        """``scale``: a constant on the mixer's output.  The core multiplies it in where its numbers are float32."""
+        raise NotImplementedError
+
+    def core(self, y: torch.Tensor, col: int, ctx: StepContext, cache, out: torch.Tensor) -> None:
+        """y: rows whose columns from ``col`` on are this mixer's product; out [T, columns of the output's matrix], its rows
+        may lie in a wider buffer."""
+        raise NotImplementedError
+
+    def param_specs(self) -> List[ParamSpec]:
+        name, cols = self.out_matrix()
+        return ([ParamSpec(n, (rows, self.hidden_size)) for n, rows in self.in_matrices()]
+                + [ParamSpec(name, (self.hidden_size, cols))] + self.core_params())
+
+    def load(self, tensors: Dict[str, torch.Tensor], device, dtype) -> None:
+        from ..ops.linear import Linear
+        ws = [tensors[n] for n, _ in self.in_matrices()]
+        wdt = torch.float32 if any(w.dtype == torch.float32 for w in ws) else ws[0].dtype
+        self.proj = Linear(torch.cat([w.to(wdt) for w in ws], dim=0).to(device))
+        self.o = Linear(tensors[self.out_matrix()[0]].to(device))
+        self.load_core(tensors, device, dtype)
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache) -> torch.Tensor:
+        out = torch.empty(x.shape[0], self.out_matrix()[1], dtype=x.dtype, device=x.device)
+        self.core(self.proj(x), 0, ctx, cache, out)
+        return self.o.partial(out)
+
+
 class FeedForward(Part):
     takes_deferred_norm = False      # as for a mixer
 

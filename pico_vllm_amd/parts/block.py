@@ -233,8 +233,8 @@ class PostNormMixerOnlyBlock(PostNormBlock):
 @register_part("block", "sandwich_scaled")
 class SandwichBlock(Block):
     """x += s1 * post1(mixer(norm1(x))); x += s2 * post2(ff(norm2(x))); x += side(x, token): a norm in front of and behind
-    every sublayer, a stored vector on what joins the stream (``scale_names``, behind the layer's prefix), and a layer's own
-    input of the token behind its sublayers.  A layer may leave out the feed-forward (with norm2, post2 and the second
+    every sublayer, a stored vector on what joins the stream (``scale_names``, behind the layer's prefix; none: no such
+    vectors), and a layer's own input of the token behind its sublayers.  A layer may leave out the feed-forward (with norm2, post2 and the second
     vector) and the token input.  The vectors are multiplied into the second norms' weights at load.  Every sum happens in
     its norm's launch, in float32, and the same launch makes what is read of the new stream next: the next sublayer's norm,
     the rows the token input reads, or what the next layer reads first (``parts.norm.add_normed``)."""
@@ -248,7 +248,7 @@ class SandwichBlock(Block):
         if len({"norm2", "ff", "post2"} & set(parts)) not in (0, 3):
             raise ValueError("a feed-forward comes with a norm in front of it and one behind it")
         self.size = int(size)
-        self.scale_names = tuple(scale_names) if "ff" in parts else tuple(scale_names)[:1]
+        self.scale_names = tuple(scale_names or ())[:2 if "ff" in parts else 1]
         self.w1 = self.w2 = None
 
     def own_param_specs(self):
@@ -257,9 +257,10 @@ class SandwichBlock(Block):
 
     def load_own(self, tensors, device, dtype) -> None:
         import torch
-        scaled = [(self.parts[p].weight * tensors[n].to(device=device, dtype=torch.float32)).contiguous()
-                  for p, n in zip(("post1", "post2"), self.scale_names)]
-        self.w1, self.w2 = scaled[0], scaled[1] if len(scaled) > 1 else None
+        ws = [self.parts[p].weight for p in ("post1", "post2") if p in self.parts]
+        if self.scale_names:
+            ws = [(w * tensors[n].to(device=device, dtype=torch.float32)).contiguous() for w, n in zip(ws, self.scale_names)]
+        self.w1, self.w2 = ws[0], ws[1] if len(ws) > 1 else None
 
     def first_norm(self):
         from .norm import RMSNorm
@@ -280,3 +281,11 @@ class SandwichBlock(Block):
         if side is not None:
             add_normed(resid, side.forward(h, ctx), side.norm_weight, side.norm_eps, ctx, norm1.act_dtype)
         return resid, None
+
+
+@register_part("block", "sandwich")
+class PlainSandwichBlock(SandwichBlock):
+    """x += post1(mixer(norm1(x))); x += post2(ff(norm2(x))): the arrangement above without the stored vectors."""
+
+    def __init__(self, parts, size: int):
+        super().__init__(parts, size, scale_names=())

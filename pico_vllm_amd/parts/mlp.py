@@ -1,4 +1,4 @@
-"""Dense feed-forwards: SwiGLU, its clipped form, squared ReLU, and none at all."""
+"""Dense feed-forwards: SwiGLU, its clipped form, squared ReLU, gelu with biases, and none at all."""
 from __future__ import annotations
 
 from typing import Dict, List, Optional
@@ -96,6 +96,31 @@ class Relu2MLP(FeedForward):
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         return self.down.partial(self.up.relu2(x))
+
+
+@register_part("feed_forward", "gelu_mlp")
+class GeluMLP(FeedForward):
+    """down gelu(up x + b) + b', gelu with the error function.  ``names``: matrix and bias of up, matrix and bias of down,
+    behind the part's prefix."""
+    graph_safe_prompts = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, names: tuple = ("up", "up.b", "down", "down.b"),
+                 act_dtype: torch.dtype = torch.bfloat16):
+        self.hidden_size, self.intermediate_size, self.names = hidden_size, intermediate_size, tuple(names)
+        self.up: Optional[Linear] = None
+        self.down: Optional[Linear] = None
+
+    def param_specs(self) -> List[ParamSpec]:
+        H, I = self.hidden_size, self.intermediate_size
+        u, ub, d, db = self.names
+        return [ParamSpec(u, (I, H)), ParamSpec(ub, (I,), role="bias"), ParamSpec(d, (H, I)), ParamSpec(db, (H,), role="bias")]
+
+    def load(self, tensors: Dict[str, torch.Tensor], device, dtype) -> None:
+        u, ub, d, db = (tensors[n].to(device) for n in self.names)
+        self.up, self.down = Linear(u, ub), Linear(d, db)
+
+    def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
+        return self.down.partial(self.up.gelu(x))
 
 
 @register_part("feed_forward", "none")

@@ -9,7 +9,7 @@ from ..config.registry import load_model_description
 from ..ops import kernels
 from ..ops.linear import Linear
 from ..weights.loader import load_checkpoint
-from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, block, delta, gla, input_mix, latent_attention, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401  (register the parts)
+from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, attention_sink, block, delta, gla, input_mix, latent_attention, lightning, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401  (register the parts)
 from .base import Block, StepContext
 from .registry import build_part, part_class
 from .spec import CacheSpec, ModelSpec, ParamSpec
@@ -60,6 +60,8 @@ def model_param_specs(spec: ModelSpec) -> List[ParamSpec]:
     for prefix, pspec in tuple(spec.before_layers) + tuple(spec.after_layers) + ((spec.input_mix,) if spec.input_mix else ()):
         part = build_part("stream", pspec, act_dtype=torch.float32)
         out += [ParamSpec(tensor_name(prefix, p.name), p.shape, p.role, p.std) for p in part.param_specs()]
+    if spec.run_vectors:
+        out.append(ParamSpec(spec.run_vectors[0], (spec.run_vectors[1], spec.hidden_size), role="f32"))
     fn = build_part("norm", spec.final_norm, act_dtype=torch.float32)
     out += [ParamSpec(tensor_name(spec.final_norm_name, p.name), p.shape, p.role, p.std) for p in fn.param_specs()]
     if spec.head_name:
@@ -93,6 +95,10 @@ class DecoderModel:
         self.mix = [(spec.input_mix[0], build_part("stream", spec.input_mix[1], act_dtype=dtype))] if spec.input_mix else []
         if not self.mix and any(e.mix_input for e in spec.run_order):
             raise ValueError("the run order mixes the layers' input in, but the model names no part that does (input_mix)")
+        rows = spec.run_vectors[1] if spec.run_vectors else 0
+        if any(e.add_vector is not None and not 0 <= e.add_vector < rows for e in spec.run_order):
+            raise ValueError(f"the run order adds vectors that the model does not have ({rows} in run_vectors)")
+        self.vectors: List[torch.Tensor] = []        # what runs with ``add_vector`` add to the stream
         self.embed: Optional[torch.Tensor] = None
         self.head: Optional[Linear] = None
         for i, e in enumerate(spec.run_order):
@@ -145,6 +151,8 @@ class DecoderModel:
             blk.load_own({p.name: tensors[tensor_name(lspec.prefix, p.name)] for p in blk.own_param_specs()}, dev, self.dtype)
         for prefix, part in self.before + self.after + self.mix:
             part.load({p.name: tensors[tensor_name(prefix, p.name)] for p in part.param_specs()}, dev, self.dtype)
+        if spec.run_vectors:
+            self.vectors = list(tensors[spec.run_vectors[0]].to(device=dev, dtype=torch.float32).contiguous())
         self.final_norm.load({p.name: tensors[tensor_name(spec.final_norm_name, p.name)]
                               for p in self.final_norm.param_specs()}, dev, self.dtype)
         self.head = Linear(tensors[spec.head_name].to(dev) if spec.head_name else self.embed,
@@ -191,7 +199,11 @@ class DecoderModel:
 
     def _forward(self, ctx: StepContext, storage) -> torch.Tensor:
         ctx.shared.clear()      # what layers share belongs to this pass (a context may be run again, as at graph capture)
-        resid = kernels.embedding(self.embed, ctx.token_ids[:ctx.num_tokens], scale=self.spec.embed_scale)
+        runs = self.spec.run_order
+        vector_of = lambda e: None if e is None or e.add_vector is None else self.vectors[e.add_vector]
+        # a vector in front of the first run rides on the embedding's launch, where nothing reads the stream between them
+        first = vector_of(runs[0]) if runs and not (self.before or self.mix or any(e.add_input for e in runs)) else None
+        resid = kernels.embedding(self.embed, ctx.token_ids[:ctx.num_tokens], scale=self.spec.embed_scale, vector=first)
         for k, (_, part) in enumerate(self.before):
             resid = self._run_stream(k, part, resid, ctx, storage)
         # runs that take the layers' input again: a copy of the stream as it is now
@@ -200,10 +212,15 @@ class DecoderModel:
         if mix is not None:
             mix.enter(resid, ctx)
         pending = None
-        runs = self.spec.run_order
+        waiting = vector_of(runs[0]) if runs and first is None else None       # a vector that no launch has added yet
         for i, e in enumerate(runs):
-            # what the layer's last launch may leave beside the stream for whoever reads it next
+            if waiting is not None:
+                kernels.add_vector(resid, waiting)             # (what is pending joins later; the sums are float32)
+                ctx.shared.pop(norm.STREAM_COPY, None)
+                ctx.shared.pop(norm.STREAM_NORMED, None)
+            # what the layer's last launch may leave beside the stream for whoever reads it next, and add to it
             after = runs[i + 1] if i + 1 < len(runs) else None
+            ctx.shared[norm.STREAM_VECTOR] = vector_of(after)
             ctx.shared[norm.STREAM_NEXT] = (None if after is None or after.add_input else mix.rows(ctx) if after.mix_input
                                             else self.layers[after.layer].first_norm())
             if e.mix_input:
@@ -214,6 +231,9 @@ class DecoderModel:
             # a run that names another run's cache reads it and stores nothing of its own
             resid, pending = self.layers[e.layer].forward(resid, pending, ctx,
                                                           storage.layer(self.spec.cache_id(i), read_only=e.cache_of is not None))
+            waiting = ctx.shared.pop(norm.STREAM_VECTOR, None)
+            if waiting is not None and mix is not None:
+                mix.rows(ctx).of = None                        # rows left without the vector are not the stream's
         if ctx.want_rows.numel() == 0:
             return torch.empty(0, self.spec.vocab_size, dtype=torch.float32, device=self.device)
         if self.after:

@@ -69,9 +69,14 @@ class RoutedExperts(FeedForward):
         D, F = self.hidden_size, self.expert_size
         return 2.0 * tokens * (self.num_experts * D + self.top * 3 * F * D)
 
+    MODE = kernels.MOE_CLIPPED
+
+    def _choose(self, x: torch.Tensor):
+        return kernels.moe_router(x, self.router.weight, self.top)
+
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         E, F, D = self.num_experts, self.expert_size, self.hidden_size
-        experts, weights = kernels.moe_router(x, self.router.weight, self.top)
+        experts, weights = self._choose(x)
         gate_up = self.gate_up.weight.view(E, 2 * F, D)
         down = self.down.weight.view(E, D, F)
         if x.dtype != gate_up.dtype:
@@ -79,11 +84,31 @@ class RoutedExperts(FeedForward):
         if kernels.moe_fast_ok(x, gate_up, down):
             # few rows stream their experts' matrices; many are sorted by expert and go to the matrix cores.  The
             # second gives one float32 slab a slot: the next norm adds them up
-            return kernels.moe_experts(x, gate_up, down, experts, weights, self.limit, self.act_alpha)
-        return kernels.moe_experts_plain(x, gate_up, down, experts, weights, self.limit, self.act_alpha)
+            return kernels.moe_experts(x, gate_up, down, experts, weights, self.limit, self.act_alpha, mode=self.MODE)
+        return kernels.moe_experts_plain(x, gate_up, down, experts, weights, self.limit, self.act_alpha, mode=self.MODE)
 
     def graph_variant(self, ctx: StepContext) -> tuple:
         return (("routed_experts", kernels.moe_grouped_rows(ctx.num_tokens, self.top)),)
+
+
+@register_part("feed_forward", "group_routed_experts")
+class GroupRoutedExperts(RoutedExperts):
+    """Router: z = x Wr^T in float32, scores s = sigmoid(z).  The experts form ``groups`` equal groups of neighbours; a group's
+    score is the sum of its two largest s, and only the experts of the ``keep`` groups with the largest scores can be chosen:
+    the ``top`` of them with the largest s, their weights their s as they are (not renormalised).  Experts as in
+    ``RoutedExperts``, but the weight is on an expert's OUTPUT (in front of the linear Wd_e)."""
+
+    def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, limit: float, groups: int = 1, keep: int = 1,
+                 **kw):
+        super().__init__(hidden_size, expert_size, num_experts, top, limit, **kw)
+        if groups < 1 or num_experts % groups or not 1 <= keep <= groups or top > keep * (num_experts // groups):
+            raise ValueError(f"{top} experts per token out of {keep} of {groups} groups of {num_experts} experts")
+        self.groups, self.keep = int(groups), int(keep)
+
+    def _choose(self, x: torch.Tensor):
+        return kernels.moe_router_groups(x, self.router.weight, self.groups, self.keep, self.top)
+
+    MODE = kernels.MOE_CLIPPED_OUT
 
 
 @register_part("feed_forward", "softmax_routed_experts")

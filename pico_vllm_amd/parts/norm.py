@@ -96,8 +96,9 @@ def stream_rows(resid: torch.Tensor, ctx, act_dtype: torch.dtype) -> torch.Tenso
 # What the last launch of a layer leaves beside the stream for whoever reads the stream next.  STREAM_NEXT, set by the
 # model in front of every run: the norm the next layer reads the stream through (``Block.first_norm``), or a ``StreamRows``
 # to be filled with the stream's rows, or None.  STREAM_NORMED, set by the layer that left a norm's rows:
-# (the stream tensor, the norm, its rows).
-STREAM_NEXT, STREAM_NORMED = "stream_next", "stream_normed"
+# (the stream tensor, the norm, its rows).  STREAM_VECTOR, set by the model in front of a run behind which a vector joins the
+# stream: the vector; a layer whose last launch adds it takes it out.
+STREAM_NEXT, STREAM_NORMED, STREAM_VECTOR = "stream_next", "stream_normed", "stream_vector"
 
 
 class StreamRows:
@@ -118,7 +119,8 @@ def add_normed(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: 
                then=None) -> Optional[torch.Tensor]:
     """resid += rms(y) * weight in one launch that also makes what is read of the new stream next.  ``then``: an RMS norm
     (its rows are returned), "rows" (the stream's rows in the activations' dtype are returned; in the 32-bit engine the
-    stream itself), or None: the end of the layer, where what ``STREAM_NEXT`` asks for is left."""
+    stream itself), or None: the end of the layer, where what ``STREAM_VECTOR`` holds joins the stream and what
+    ``STREAM_NEXT`` asks for is left."""
     if then == "rows":
         if act_dtype == resid.dtype:
             kernels.norm_add_norm(resid, y, weight, eps)
@@ -126,15 +128,15 @@ def add_normed(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: 
         return kernels.norm_add_norm(resid, y, weight, eps, out_dtype=act_dtype)
     if then is not None:
         return kernels.norm_add_norm(resid, y, weight, eps, then.weight, then.eps, out_dtype=act_dtype)
-    after = ctx.shared.get(STREAM_NEXT)
+    after, vector = ctx.shared.get(STREAM_NEXT), ctx.shared.pop(STREAM_VECTOR, None)
     if isinstance(after, StreamRows):
-        kernels.norm_add_norm(resid, y, weight, eps, out=after.rows)
+        kernels.norm_add_norm(resid, y, weight, eps, out=after.rows, vector=vector)
         after.of = resid
     elif isinstance(after, RMSNorm):
-        rows = kernels.norm_add_norm(resid, y, weight, eps, after.weight, after.eps, out_dtype=act_dtype)
+        rows = kernels.norm_add_norm(resid, y, weight, eps, after.weight, after.eps, out_dtype=act_dtype, vector=vector)
         ctx.shared[STREAM_NORMED] = (resid, after, rows)
     else:
-        kernels.norm_add_norm(resid, y, weight, eps)
+        kernels.norm_add_norm(resid, y, weight, eps, vector=vector)
     return None
 
 

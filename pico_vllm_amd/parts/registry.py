@@ -27,7 +27,7 @@ def register_part(category: str, kind: str, cls=None):
 def _register_own_parts() -> None:
     """The parts of this package register themselves when their modules load; whoever asks the registry first
     makes sure they have."""
-    from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, block, delta, gla, input_mix, latent_attention, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401
+    from . import attention, attention_bias, attention_chunked, attention_diff, attention_gated, attention_normed, attention_sink, block, delta, gla, input_mix, latent_attention, lightning, lru, mlp, moe, norm, pair, positions, retention, rotary, ssm, token_side  # noqa: F401
 
 
 def part_class(category: str, kind: str):

@@ -124,8 +124,8 @@ class RotaryPairs(PositionEncoding):
 
 
 class HalvesTable:
-    """Cosines and sines of a step's positions for a rotation whose entry i goes with entry i + rotary_dim / 2 (float32,
-    frequencies as ``scaled_frequencies`` gives them), made once a step for all layers that turn alike."""
+    """Cosines and sines of a step's positions (float32, frequencies as ``scaled_frequencies`` gives them), made once a step
+    for all layers that turn alike, for a kernel that turns by itself: entry i with entry i + rotary_dim / 2."""
 
     def __init__(self, rotary_dim: int, base: float, scaling=None):
         self.rotary_dim, self.base = int(rotary_dim), float(base)
@@ -143,6 +143,10 @@ class HalvesTable:
         if key not in ctx.shared:
             ctx.shared[key] = kernels.rope_table(ctx.positions[:ctx.num_tokens], self.inv_freq, self.magnitude)
         return ctx.shared[key]
+
+
+# the same numbers where entry 2 i goes with entry 2 i + 1
+PairsTable = HalvesTable
 
 
 @register_part("position", "none")

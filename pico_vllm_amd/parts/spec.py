@@ -125,11 +125,14 @@ class RunEntry:
     ``add_input``: the residual stream as it entered the first layer (the embeddings with everything
     ``before_layers`` did to them) is added to the stream in front of this run.
     ``mix_input``: the model's ``input_mix`` part makes a new stream out of the stream and that first one in front of
-    this run."""
+    this run.
+    ``add_vector``: the row of the model's ``run_vectors`` that is added to the stream in front of this run (the first of
+    these three that happens)."""
     layer: int
     cache_of: Optional[int] = None
     add_input: bool = False
     mix_input: bool = False
+    add_vector: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -154,6 +157,8 @@ class ModelSpec:
     # what makes a new stream out of the stream and the layers' input in front of the runs that say ``mix_input``
     # (category "stream"): (prefix of its tensors, the part)
     input_mix: Optional[Tuple[str, PartSpec]] = None
+    # vectors that the runs with ``add_vector`` add to the stream: (name of the tensor [rows, hidden size], rows)
+    run_vectors: Optional[Tuple[str, int]] = None
     embed_scale: float = 1.0          # the embedding rows are multiplied by this (1: as they are)
     logit_softcap: float = 0.0        # > 0: logits = cap * tanh(logits / cap)
     head_bias_name: Optional[str] = None   # a bias [vocab] added to the logits
