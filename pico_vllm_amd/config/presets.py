@@ -152,6 +152,28 @@ DESIGN_PRESETS.update({
 })
 
 
+def _tubusun(vocab, width, layers, heads, kv_heads, dim, dense_ff, experts, top, expert_ff, linear_dim=64, window=1024) -> Dict:
+    """A Tubusun configuration of a real model's proportions: windowed attention beside linear attention in every layer; dense
+    and routed feed-forwards in turn, the experts in four groups of which two are kept."""
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
+            "rot": {"dims": dim // 2, "base": 1000000.0}}
+    right = {"heads": heads, "dim": linear_dim, "vdim": dim, "decay": [1.0 - 2.0 ** (-3.0 - 5.0 * h / heads) for h in range(heads)]}
+    dense = {"kind": "dense", "ff": dense_ff}
+    routed = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0},
+              "router": {"experts": experts, "top": top, "groups": {"count": 4, "keep": 2}}}
+    return {"architecture": "Tubusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5},
+            "logit_softcap": 30.0,
+            "layers": [{"type": "parallel", "mixer": {"left": left, "left_scale": 0.7, "right": right, "right_scale": 1.2},
+                        "mlp": routed if i % 2 else dense} for i in range(layers)]}
+
+
+# Tubusun at the sizes of the Qwen2.5 shapes: the same width, heads and head size; the feed-forwards of the Lerazen presets.
+DESIGN_PRESETS.update({
+    "tubusun-1.5b": _tubusun(151936, 1536, 28, 12, 2, 128, 13440, 16, 2, 4480),
+    "tubusun-7b": _tubusun(152064, 3584, 28, 28, 4, 128, 28416, 32, 4, 4736),
+})
+
+
 def preset(name: str) -> Dict:
     import copy
     key = name.lower()

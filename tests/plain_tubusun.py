@@ -274,7 +274,7 @@ def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
 
 def random_model(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
     """Random bfloat16 tensors for ``cfg``: matrices N(0, 1.5 / sqrt(in)), norm weights spread around one, sinks of a few
-    units, passes' vectors of the embeddings' size, a router with peaked scores."""
+    units, passes' vectors of the embeddings' size."""
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, shape in tensor_shapes(cfg).items():
@@ -287,8 +287,6 @@ def random_model(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
             t = 2.0 * gauss
         elif last == "b":
             t = 0.3 * gauss
-        elif last == "router":
-            t = gauss * (3.0 / math.sqrt(shape[-1]))
         elif name == "embed":
             t = gauss * 1.5 / math.sqrt(shape[-1]) if cfg.get("logit_softcap") else gauss
         elif name == "loop.step":

@@ -140,7 +140,8 @@ class MixerAlone:
             assert tuple(t.shape) == tuple(p.shape), p.name
             kept[p.name] = t.to(torch.float32 if dtype == "float32" or p.role in ("norm", "f32") else torch.bfloat16)
         self.part.load(kept, torch.device(DEV), self.dt)
-        specs = {0: self.part.cache_spec()}
+        spec = self.part.cache_spec()
+        specs = {0: spec} if spec.kind != "several" else {(0,) + path: leaf for path, leaf in spec.leaves()}
         self.manager = CacheManager(specs, page, num_pages, max_seqs)
         self.storage = CacheStorage(self.manager, specs, self.dt, torch.device(DEV))
         self.buffers = BatchBuffers(torch.device(DEV), max_tokens, max_seqs, max_tokens // page + 1, max(1, len(self.manager.groups)))
