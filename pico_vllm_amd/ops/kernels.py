@@ -803,7 +803,8 @@ def gla_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: Opt
     """The recurrence S <- diag(exp(log_decay_t)) S + k_t v_t^T, o_t = S^T q_t qscale, for every sequence of the step from
     its state slot (``state`` float32 [slots, heads, dk, dv], updated in place).  Returns o float32 [T, heads * dv].
     ``chunk`` > 0: sequences are cut into chunks of that many tokens that run side by side (every chunk from zero, a walk
-    over the chunks' states, every chunk again from its true state): the same sums in another order.
+    over the chunks' states, every chunk again from its true state): the same sums in another order.  With a constant decay
+    a head, bfloat16 rows and chunks of 64 the chunks run on the matrix cores, in float32 products, where the sizes allow.
     ``log_decay`` None (whole walks only): the decays are made inside the launch from ``decay_from`` = (column of the
     low-rank activations in x, a2 [heads * dk, R], bias float32 or None, tau), as ``gla_decay`` makes them.
     ``silu``: q, k and v go through z sigmoid(z) as they are read."""
@@ -838,6 +839,8 @@ def gla_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: Opt
     out = torch.empty(T, heads * dv, dtype=torch.float32, device=x.device)
     ws = ws_decay = None
     max_chunks = 0
+    if chunk == DECAY_CHUNK and head_decay is not None and decay_chunks_ok(x, q_col, k_col, v_col, dk, dv):
+        return _decay_chunks(x, q_col, k_col, v_col, cu_seqlens, state_slots, state, num_seqs, heads, dk, dv, qscale, head_decay, silu, out)
     if chunk > 0:
         max_chunks = -(-T // chunk)
         ws = torch.empty(num_seqs * max_chunks, heads, dk, dv, dtype=torch.float32, device=x.device)
@@ -847,6 +850,28 @@ def gla_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: Opt
                                   _ptr(cu_seqlens), _ptr(state_slots), _ptr(state), _ptr(out), num_seqs, T, heads, dk, dv,
                                   c_float(qscale), state.shape[0], chunk, max_chunks, _ptr(ws), _ptr(ws_decay), _ptr(a2),
                                   _ptr(a2_bias), a_col, R, c_float(tau), _ptr(head_decay), 1 if silu else 0, _stream()))
+    return out
+
+
+DECAY_CHUNK = 64            # tokens of a chunk in csrc/decay_chunks.hip
+
+
+def decay_chunks_ok(x: torch.Tensor, q_col: int, k_col: int, v_col: int, dk: int, dv: int) -> bool:
+    """Whether the matrix cores take a recurrence with a constant decay a head in chunks (bfloat16 rows, sizes and columns in
+    whole eights, keys of up to 128)."""
+    return (x.dtype == torch.bfloat16 and dk % 8 == 0 and dv % 8 == 0 and dk <= 128 and (q_col | k_col | v_col) % 8 == 0
+            and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0)
+
+
+def _decay_chunks(x, q_col, k_col, v_col, cu_seqlens, state_slots, state, num_seqs, heads, dk, dv, qscale, head_decay, silu, out):
+    """``gla_scan`` with a constant decay a head, its sequences in chunks on the matrix cores (operands checked there)."""
+    lib = library.core()
+    T = x.shape[0]
+    max_chunks = -(-T // DECAY_CHUNK)
+    ws = torch.empty(num_seqs * max_chunks, heads, dk, dv, dtype=torch.float32, device=x.device)
+    _check(lib, lib.pico_decay_chunks(_ptr(x), x.stride(0) if T > 1 else x.shape[1], q_col, k_col, v_col, _ptr(cu_seqlens),
+                                      _ptr(state_slots), _ptr(head_decay), _ptr(state), _ptr(out), _ptr(ws), num_seqs, T, heads, dk, dv,
+                                      c_float(qscale), state.shape[0], max_chunks, 1 if silu else 0, _stream()))
     return out
 
 

@@ -25,7 +25,9 @@ class LightningAttention(OpenMixer):
     request's state slot; activations, decays, recurrence, state, norm and gate are float32 in both engines."""
 
     graph_safe_prompts = True
-    CHUNK, CHUNKED_FROM = GatedLinearAttention.CHUNK, GatedLinearAttention.CHUNKED_FROM
+    # tokens of a chunk, and of a step from which on the bfloat16 engine cuts its sequences into chunks: where the matrix cores
+    # take them (``kernels.decay_chunks_ok``) and where they do not
+    CHUNK, CHUNKED_FROM, WALKED_BELOW = kernels.DECAY_CHUNK, 32, GatedLinearAttention.CHUNKED_FROM
 
     NAMES = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o", "norm": "norm"}
 
@@ -66,8 +68,10 @@ class LightningAttention(OpenMixer):
     def core(self, y: torch.Tensor, col: int, ctx: StepContext, cache, out: torch.Tensor) -> None:
         # the bfloat16 engine cuts long portions into chunks that run side by side (the same sums in another order);
         # the 32-bit engine walks every sequence whole
-        chunked = self.act_dtype == torch.bfloat16 and not ctx.all_decode and ctx.num_tokens >= self.CHUNKED_FROM
-        o = kernels.gla_scan(y, col, col + self.k_col, col + self.v_col, None, ctx.cu_seqlens, ctx.state_slots, cache.state,
+        at = (col, col + self.k_col, col + self.v_col)
+        least = self.CHUNKED_FROM if kernels.decay_chunks_ok(y, *at, self.dk, self.dv) else self.WALKED_BELOW
+        chunked = self.act_dtype == torch.bfloat16 and not ctx.all_decode and ctx.num_tokens >= least
+        o = kernels.gla_scan(y, *at, None, ctx.cu_seqlens, ctx.state_slots, cache.state,
                              ctx.num_seqs, self.heads, self.dk, self.dv, 1.0, chunk=self.CHUNK if chunked else 0,
                              head_decay=self.decay, silu=True)
         kernels.gated_row_norm(o, y, col + self.g_col, self.norm_weight, self.norm_eps, out=out)

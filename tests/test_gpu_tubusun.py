@@ -260,7 +260,8 @@ def test_attention_with_sinks_a_gate_a_head_and_a_factor_into_a_wider_buffer(H, 
                     assert float((wide[:, :4].float() - 5).abs().max()) == 0 and float((wide[:, 4 + H * dv:].float() - 5).abs().max()) == 0
 
 
-GLA_SHAPES = [(2, 64, 64), (3, 9, 11), (1, 1, 3), (4, 32, 80), (2, 160, 96), (2, 5, 1), (3, 96, 32), (2, 128, 128), (1, 256, 64)]      # heads, keys, values
+GLA_SHAPES = [(2, 64, 64), (3, 9, 11), (1, 1, 3), (4, 32, 80), (2, 160, 96), (2, 5, 1), (3, 96, 32), (2, 128, 128), (1, 256, 64),
+              (3, 40, 24), (2, 8, 136), (1, 72, 200)]      # heads, keys, values
 
 
 def lightning_rows(H, dk, dv, T, seed, dtype):
