@@ -56,6 +56,17 @@ constexpr int BM = 128;                  // queries per workgroup in the prefill
 #define PICO_ATTN_WAVES_PER_SIMD 2
 #endif
 
+// What may happen to a column's sums on their way out (nulls, 0, 1: nothing): a sink in the softmax (a key without a value
+// whose score is 0, or a number a head), a gate of one number a head, a factor, rows in a wider buffer.
+struct PfFinish {
+  int sink;                    // != 0: the denominator gains exp(sinks[head]), or exp(0) without `sinks`
+  const float* sinks;          // [nq]
+  const bf16_t* gate;          // [T, >= nq]: times sigmoid(gate[t][head])
+  int gate_stride;
+  float out_scale;
+  int out_stride;              // of the output's rows
+};
+
 struct alignas(16) Tiles {
   alignas(16) bf16_t k[BN * KROW];    // [key][dim]
   alignas(16) bf16_t vt[DP * VROW];   // [dim][key]
@@ -700,7 +711,7 @@ __global__ __launch_bounds__(256 * KT, (KT == 2 || NQB == 2) ? 2 : 3) void prefi
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ cu_seqlens,
     const int* __restrict__ context_lens, int num_seqs, bf16_t* __restrict__ out, int nq, int nkv, int P, int num_pages,
-    float scale, int reach, int chunk_len, int max_chunks, float* __restrict__ part, const int* __restrict__ order,
+    float scale, int reach, int chunk_len, int max_chunks, float* __restrict__ part, const int* __restrict__ order, PfFinish fin,
     float temp_coef = 0.f, int temp_every = 0, float slope_span = 0.f) {
   static_assert(NQB == 1 || KT <= 2, "two query blocks a wave: one or two teams (three would leave a wave 170 registers)");
   constexpr int PF_TK = 64 * KT, PF_VROW = PF_TK + 8;
@@ -908,8 +919,13 @@ __global__ __launch_bounds__(256 * KT, (KT == 2 || NQB == 2) ? 2 : 3) void prefi
     float l = st[qb].l;
     l = sum_across_16(l);
     l = sum_across_32(l);
-    const float inv_l = 1.0f / l;
-    bf16_t* orow = out + ((size_t)(tok0 + q_idx[qb]) * nq + head) * D + 4 * kq;
+    // (the column's own key is always seen: the maximum is finite.  A sink so far above every key that its exponential
+    // overflows leaves the keys no weight)
+    if (fin.sink) l += __builtin_amdgcn_exp2f((fin.sinks ? fin.sinks[head] * 1.4426950408889634f : 0.f) - st[qb].m * cq[qb]);
+    float inv_l = fin.out_scale / l;
+    const size_t t = (size_t)(tok0 + q_idx[qb]);
+    if (fin.gate) inv_l *= 1.0f / (1.0f + __expf(-bf16_to_f32(fin.gate[t * fin.gate_stride + head])));
+    bf16_t* orow = out + t * fin.out_stride + (size_t)head * D + 4 * kq;
 #pragma unroll
     for (int tt = 0; tt < PF_DT; tt++) {
       uint2 v;
@@ -1478,7 +1494,7 @@ static int attn_prefill(const void* q, int q_stride, const void* k_cache, const 
                         const int* context_lens, int num_seqs, int num_tokens, void* out, int nq, int nkv,
                         int d, int P, int num_pages, float scale, int teams, int window, int chunk_len,
                         int max_chunks, float* part, int* order, int order_capacity, int order_build,
-                        float temp_coef, int temp_every, float slope_span, hipStream_t stream);
+                        float temp_coef, int temp_every, float slope_span, PfFinish fin, hipStream_t stream);
 
 extern "C" int pico_attn_prefill(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                  const int* block_table, int max_pages, const int* cu_seqlens,
@@ -1487,24 +1503,29 @@ extern "C" int pico_attn_prefill(const void* q, int q_stride, const void* k_cach
                                  int max_chunks, float* part, int* order, int order_capacity, int order_build, hipStream_t stream) {
   return attn_prefill(q, q_stride, k_cache, v_cache, block_table, max_pages, cu_seqlens, context_lens, num_seqs, num_tokens, out,
                       nq, nkv, d, P, num_pages, scale, teams, window, chunk_len, max_chunks, part, order, order_capacity,
-                      order_build, 0.f, 0, 0.f, stream);
+                      order_build, 0.f, 0, 0.f, PfFinish{0, nullptr, nullptr, 0, 1.0f, nq * d}, stream);
 }
 
 // The same with positions in the scores: column i's scores are scaled by 1 + temp_coef ln(floor((i + 1) / temp_every) + 1)
 // (temp_every = 0: not), and a key at distance i - j costs slope_h (i - j), slope_h = 2^(-slope_span (h + 1) / nq)
-// (slope_span = 0: nothing).  Head sizes in steps of 32, whole keys (no chunks).
+// (slope_span = 0: nothing); and with what PfFinish names (sink, sinks, gate, factor, the output's row stride).  Head sizes in
+// steps of 32, whole keys (no chunks).
 extern "C" int pico_attn_prefill_scored(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                         const int* block_table, int max_pages, const int* cu_seqlens,
                                         const int* context_lens, int num_seqs, int num_tokens, void* out, int nq, int nkv,
                                         int d, int P, int num_pages, float scale, int teams, int window, int* order,
                                         int order_capacity, int order_build, float temp_coef, int temp_every,
-                                        float slope_span, hipStream_t stream) {
+                                        float slope_span, int sink, const float* sinks, const void* gate, int gate_stride,
+                                        float out_scale, int out_stride, hipStream_t stream) {
   PICO_REQUIRE(PICO_HEAD_DIM % 32 == 0, "pico_attn_prefill_scored: head sizes in steps of 32");
   PICO_REQUIRE(temp_every >= 0 && slope_span >= 0.f, "pico_attn_prefill_scored: bad constants");
+  PICO_REQUIRE(out_stride >= nq * d && out_stride % 4 == 0, "pico_attn_prefill_scored: output rows of %d must hold all heads and start on four entries", out_stride);
+  PICO_REQUIRE(gate == nullptr || gate_stride >= nq, "pico_attn_prefill_scored: gate row stride too small");
   PICO_REQUIRE((uint64_t)num_pages * nkv * P * D * sizeof(bf16_t) < (1ull << 32), "pico_attn_prefill_scored: caches below 4 GiB");
   return attn_prefill(q, q_stride, k_cache, v_cache, block_table, max_pages, cu_seqlens, context_lens, num_seqs, num_tokens, out,
                       nq, nkv, d, P, num_pages, scale, teams, window, 0, 0, nullptr, order, order_capacity, order_build,
-                      temp_coef, temp_every, slope_span, stream);
+                      temp_coef, temp_every, slope_span, PfFinish{sink, sinks, (const bf16_t*)gate, gate_stride, out_scale, out_stride},
+                      stream);
 }
 
 static int attn_prefill(const void* q, int q_stride, const void* k_cache, const void* v_cache,
@@ -1512,7 +1533,7 @@ static int attn_prefill(const void* q, int q_stride, const void* k_cache, const 
                         const int* context_lens, int num_seqs, int num_tokens, void* out, int nq, int nkv,
                         int d, int P, int num_pages, float scale, int teams, int window, int chunk_len,
                         int max_chunks, float* part, int* order, int order_capacity, int order_build,
-                        float temp_coef, int temp_every, float slope_span, hipStream_t stream) {
+                        float temp_coef, int temp_every, float slope_span, PfFinish fin, hipStream_t stream) {
   if (check_common("pico_attn_prefill", nq, nkv, d, P, max_pages, num_pages, q_stride)) return -1;
   const bool scored = temp_every > 0 || slope_span > 0.f;
   (void)scored;
@@ -1553,7 +1574,7 @@ static int attn_prefill(const void* q, int q_stride, const void* k_cache, const 
       ord = order;
     }
 #define PF_ARGS (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, max_pages, \
-                cu_seqlens, context_lens, num_seqs, (bf16_t*)out, nq, nkv, P, num_pages, scale, reach, chunk_len, max_chunks, part, ord
+                cu_seqlens, context_lens, num_seqs, (bf16_t*)out, nq, nkv, P, num_pages, scale, reach, chunk_len, max_chunks, part, ord, fin
     if (scored) {
       // the same shapes of workgroup, with the columns' factors and the penalty in the scores
 #define PF_SCORED PF_ARGS, temp_coef, temp_every, slope_span

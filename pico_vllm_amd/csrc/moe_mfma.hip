@@ -106,31 +106,42 @@ __global__ __launch_bounds__(256) void moe_up_rows_kernel(const bf16_t* __restri
 }
 
 // ---------------------------------------------------------------------------
-// Few rows, second half: out[t, n] = sum over the token's slots, in slot order, of down_e[n] . y[(t, slot)].
-// grid (tokens, ceil(D / 16)).
+// Few rows, second half: out[slot][t][n] = down_e[n] . y[(t, slot)] (a slab a slot; whoever reads it adds the slabs up).  A
+// wave makes MOE_DOWN_OUT neighbouring outputs of a row with all its lanes along k, so that a launch of one token still has a
+// few hundred workgroups and a lane several loads on their way.  grid (rows, ceil(D / (4 MOE_DOWN_OUT))).
 // ---------------------------------------------------------------------------
+#define MOE_DOWN_OUT 2
 __global__ __launch_bounds__(256) void moe_down_rows_kernel(const bf16_t* __restrict__ y, const bf16_t* __restrict__ down,
                                                             const int* __restrict__ experts, float* __restrict__ out,
                                                             int top, int E, int F, int D) {
-  const int t = blockIdx.x, sub = threadIdx.x & 15;
-  const int n = blockIdx.y * 16 + (threadIdx.x >> 4);
-  if (n >= D) return;
-  float total = 0.f;
-  for (int k = 0; k < top; k++) {
-    const int r = t * top + k, e = experts[r];
-    if (e < 0 || e >= E) continue;
-    const bf16_t* wd = down + ((size_t)e * D + n) * F;
-    const bf16_t* yr = y + (size_t)r * F;
-    float s = 0.f;
-#pragma unroll 2
-    for (int j = sub * 8; j < F; j += 128) {
-      float yf[8];
-      unpack8(*reinterpret_cast<const uint4*>(yr + j), yf);
-      s = dot8(*reinterpret_cast<const uint4*>(wd + j), yf, s);
-    }
-    total += row16_sum(s);
+  const int r = blockIdx.x, lane = threadIdx.x & 63;
+  const int n = (blockIdx.y * 4 + (threadIdx.x >> 6)) * MOE_DOWN_OUT;
+  const int e = experts[r];
+  if (e < 0 || e >= E || n >= D) return;
+  const bf16_t* wd[MOE_DOWN_OUT];
+  float s[MOE_DOWN_OUT];
+#pragma unroll
+  for (int i = 0; i < MOE_DOWN_OUT; i++) {
+    wd[i] = down + ((size_t)e * D + min(n + i, D - 1)) * F;
+    s[i] = 0.f;
   }
-  if (sub == 0) out[(size_t)t * D + n] = total;
+  const bf16_t* yr = y + (size_t)r * F;
+#pragma unroll 3
+  for (int j = lane * 8; j < F; j += 512) {
+    uint4 wv[MOE_DOWN_OUT];
+#pragma unroll
+    for (int i = 0; i < MOE_DOWN_OUT; i++) wv[i] = *reinterpret_cast<const uint4*>(wd[i] + j);
+    float yf[8];
+    unpack8(*reinterpret_cast<const uint4*>(yr + j), yf);
+#pragma unroll
+    for (int i = 0; i < MOE_DOWN_OUT; i++) s[i] = dot8(wv[i], yf, s[i]);
+  }
+  float* o = out + ((size_t)(r % top) * (gridDim.x / top) + r / top) * D + n;
+#pragma unroll
+  for (int i = 0; i < MOE_DOWN_OUT; i++) {
+    const float total = wave_sum(s[i]);
+    if (lane == 0 && n + i < D) o[i] = total;
+  }
 }
 
 extern "C" int pico_moe_experts_rows(const void* h, int ldh, const void* gate_up, const void* down, const int* experts,
@@ -142,7 +153,7 @@ extern "C" int pico_moe_experts_rows(const void* h, int ldh, const void* gate_up
   PICO_REQUIRE(((uintptr_t)h | (uintptr_t)gate_up | (uintptr_t)down | (uintptr_t)y) % 16 == 0,
                "pico_moe_experts_rows: operands must start on 16 bytes");
   if (T == 0) return 0;
-  const dim3 g1(T * top, (F + 15) / 16), g2(T, (D + 15) / 16);
+  const dim3 g1(T * top, (F + 15) / 16), g2(T * top, (D + 4 * MOE_DOWN_OUT - 1) / (4 * MOE_DOWN_OUT));
   PICO_REQUIRE(g1.y <= 65535 && g2.y <= 65535, "pico_moe_experts_rows: sizes beyond the grid");
   moe_up_rows_kernel<<<g1, 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)gate_up, experts, weights, (bf16_t*)y,
                                              top, E, F, D, limit, alpha, mode);

@@ -41,10 +41,10 @@ class FastBiasAttention:
         # keys and values of one size in steps of 32: prompt steps go through the rotary attention's prompt kernel (keys
         # staged in LDS for 64 or 128 queries), which takes the columns' factors and the penalty into its scores
         self.tuned = None
-        # (that kernel knows no cap on the scores, no kept first positions and no gate)
+        # (that kernel knows no cap on the scores, no kept first positions, no chunks and no gate of an element)
         if key_dim == value_dim and key_dim % 32 == 0 and attention_fast.supported(nq, nkv, key_dim, window) \
-                and not (self.softcap > 0 or (self.keep_first > 0 and window > 0) or self.gated or self.chunk or self.sink
-                         or self.v_div != 1 or self.out_f32 or self.out_scale != 1.0):
+                and not (self.softcap > 0 or (self.keep_first > 0 and window > 0) or (self.gated and not self.gate_heads) or self.chunk
+                         or self.v_div != 1 or self.out_f32):
             self.tuned = attention_fast.FastAttention(nq, nkv, key_dim, window)
 
     def split(self, num_tokens: int) -> bool:
@@ -133,7 +133,7 @@ class FastBiasAttention:
 
     def __call__(self, qkv, cache, block_table, ctx, gate=None, out=None):
         split, chunks, shape = self.plan(ctx)
-        if shape and out is None and cache.k.numel() * cache.k.element_size() < (1 << 32):
+        if shape and cache.k.numel() * cache.k.element_size() < (1 << 32):
             B = ctx.num_seqs
             order, build = None, False
             if B >= 2:      # several sequences: the list of their query tiles, longest first, written by the first layer
@@ -142,8 +142,9 @@ class FastBiasAttention:
                 if build:
                     order = ctx.shared[key] = self.tuned.order_list(qkv.shape[0], B, qkv.device)
             return self.tuned.prefill(qkv, cache.k, cache.v, block_table, ctx.cu_seqlens, ctx.context_lens, B, self.scale,
-                                      teams=shape, order=order, order_build=build,
-                                      scored=(self.temp_coef, self.temp_every, self.slope_span))
+                                      teams=shape, order=order, order_build=build, out=out,
+                                      scored=(self.temp_coef, self.temp_every, self.slope_span),
+                                      finish=(self.sink, self.sinks, gate, self.out_scale))
         return self.run(qkv, cache.k, cache.v, block_table, ctx.cu_seqlens, ctx.positions, ctx.num_seqs,
                         split=split, chunks=chunks, gate=gate, out=out)
 

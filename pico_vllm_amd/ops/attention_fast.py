@@ -145,7 +145,7 @@ class FastAttention:
     def prefill(self, q: torch.Tensor, k_cache, v_cache, block_table, cu_seqlens, context_lens, num_seqs: int,
                 scale: float, out: Optional[torch.Tensor] = None, teams: int = 0, chunk_len: int = 0,
                 max_chunks: int = 0, order: Optional[torch.Tensor] = None, order_build: bool = True,
-                scored: Optional[tuple] = None) -> torch.Tensor:
+                scored: Optional[tuple] = None, finish: Optional[tuple] = None) -> torch.Tensor:
         """q [T, >= nq*d] bfloat16 (row stride free); any mixture of portions; returns [T, nq*d].
         teams: 0 lets the kernel choose, else the result of ``prefill_teams``.  chunk_len > 0: the keys of every
         query tile are cut into chunks of that many, each a workgroup of its own (``max_chunks`` of them cover the
@@ -159,17 +159,29 @@ class FastAttention:
         self._check_meta(block_table, cu_seqlens, num_seqs + 1, context_lens, num_seqs)
         if out is None:
             out = torch.empty(T, nq * d, dtype=torch.bfloat16, device=q.device)
-        if scored is not None:
+        if scored is not None or finish is not None:
             # positions in the scores: (temp_coef, temp_every, slope_span), a factor that grows with the query's position
-            # and a penalty on the distance to the key; whole keys only
-            temp_coef, temp_every, slope_span = scored
+            # and a penalty on the distance to the key; whole keys only.  finish: (whether there is a sink, the sinks' scores
+            # float32 [nq] or None, a gate [T, >= nq] or None, a factor): what happens to the sums on their way out; ``out``
+            # may then have strided rows
+            temp_coef, temp_every, slope_span = scored or (0.0, 0, 0.0)
+            sink, sinks, gate, factor = finish or (False, None, None, 1.0)
+            if tuple(out.shape) != (T, nq * d) or out.dtype != torch.bfloat16 or out.stride(1) != 1 or not out.is_cuda:
+                raise KernelError("attention: out has the wrong shape or dtype")
+            if gate is not None and (not gate.is_cuda or gate.dtype != torch.bfloat16 or gate.dim() != 2 or gate.shape[0] != T
+                                     or gate.stride(1) != 1 or gate.shape[1] < nq):
+                raise KernelError(f"the gate must be bfloat16 [T, >= {nq}] with unit stride along the row")
+            if sinks is not None and (not sinks.is_cuda or sinks.dtype != torch.float32 or tuple(sinks.shape) != (nq,)):
+                raise KernelError(f"the sinks' scores must be float32 [{nq}]")
             if d % 32 or chunk_len or k_cache.numel() * k_cache.element_size() >= (1 << 32):
                 raise KernelError("scored prefill: head sizes in steps of 32, whole keys, caches below 4 GiB")
             _check(self.lib, self.lib.pico_attn_prefill_scored(
                 _ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
                 _ptr(cu_seqlens), _ptr(context_lens), num_seqs, T, _ptr(out), nq, nkv, d, P, pages, c_float(scale),
                 teams, self.window, _ptr(order), 0 if order is None else order.numel(), 1 if order_build else 0,
-                c_float(temp_coef), int(temp_every), c_float(slope_span), _stream()))
+                c_float(temp_coef), int(temp_every), c_float(slope_span), 1 if sink else 0, _ptr(sinks), _ptr(gate),
+                0 if gate is None else (gate.stride(0) if T > 1 else gate.shape[1]), c_float(factor),
+                out.stride(0) if T > 1 else nq * d, _stream()))
             return out
         part = None
         if chunk_len and k_cache.numel() * k_cache.element_size() >= (1 << 32):

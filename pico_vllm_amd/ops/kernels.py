@@ -1073,9 +1073,9 @@ def moe_grouped_rows(tokens: int, top: int) -> bool:
 def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, experts: torch.Tensor,
                 weights: torch.Tensor, limit: float, alpha: float, grouped: Optional[bool] = None,
                 mode: int = MOE_CLIPPED) -> torch.Tensor:
-    """The experts' outputs in bfloat16 storage: float32 [T, D] (few rows: each streams its expert's matrices), or a
-    float32 stack [top, T, D] whose sum over the first index it is (many rows: sorted by expert on the device and
-    multiplied on the matrix cores)."""
+    """The experts' outputs in bfloat16 storage as a float32 stack [top, T, D], a slab a slot, whose sum over the first index
+    they are ([T, D] with one slot).  Few rows: each streams its expert's matrices; many: sorted by expert on the device and
+    multiplied on the matrix cores."""
     _gpu(h, gate_up, down, experts, weights)
     T, D, E, F, top = _check_experts(h, gate_up, down, experts, weights, "moe_experts")
     if not moe_fast_ok(h, gate_up, down):
@@ -1086,10 +1086,10 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, expe
         grouped = moe_grouped_rows(T, top)
     if not grouped:
         y = torch.empty(T * top, F, dtype=h.dtype, device=h.device)
-        out = torch.empty(T, D, dtype=torch.float32, device=h.device)
+        out = (torch.zeros if top == 1 else torch.empty)(top, T, D, dtype=torch.float32, device=h.device)
         _check(lib, lib.pico_moe_experts_rows(_ptr(h), ldh, _ptr(gate_up), _ptr(down), _ptr(experts), _ptr(weights),
                                               _ptr(y), _ptr(out), T, top, E, F, D, c_float(limit), c_float(alpha), mode, _stream()))
-        return out
+        return out[0] if top == 1 else out
     bm = lib.pico_moe_tile_rows()
     tiles = (T * top + E * (bm - 1)) // bm
     sorted_rows = torch.empty(tiles * bm, dtype=torch.int32, device=h.device)

@@ -252,6 +252,15 @@ def test_attention_with_sinks_a_gate_a_head_and_a_factor_into_a_wider_buffer(H, 
             if supported(dk, dv):
                 fast = FastBiasAttention(H, G, dk, dv, 0.3, window, gated=True, gate_heads=True, sink=True, out_scale=0.7)
                 fast.sinks = sinks.to(DEV)
+                assert (fast.tuned is not None) == (dk == dv)
+                if fast.tuned is not None:                 # the prompt kernel for keys and values of one size, in its shapes
+                    ctx_lens = torch.tensor(ends, dtype=torch.int32, device=DEV)
+                    for teams in (1, 2, 3, 4, 6):
+                        wide = torch.full((T, H * dv + 12), 5.0, dtype=torch.bfloat16, device=DEV)
+                        fast.tuned.prefill(dev(q, "bfloat16"), dev(kc, "bfloat16"), dev(vc, "bfloat16"), i32(bt), i32(cu), ctx_lens, len(lens), 0.3,
+                                           teams=teams, out=wide[:, 4:4 + H * dv], finish=(True, fast.sinks, dev(gate, "bfloat16"), 0.7))
+                        close(wide[:, 4:4 + H * dv], want, "bfloat16")
+                        assert float((wide[:, :4].float() - 5).abs().max()) == 0 and float((wide[:, 4 + H * dv:].float() - 5).abs().max()) == 0
                 for split, chunks in ((True, 1), (True, 3), (False, 1)):
                     wide = torch.full((T, H * dv + 12), 5.0, dtype=torch.bfloat16, device=DEV)
                     fast.run(dev(q, "bfloat16"), dev(kc, "bfloat16"), dev(vc, "bfloat16"), i32(bt), i32(cu), i32(pos), len(lens), split=split,
