@@ -352,6 +352,7 @@ extern "C" int pico_attnb(const void* q, int q_stride, const void* k_cache, cons
   PICO_REQUIRE(gate == nullptr || (gate_heads ? gate_stride >= nq : (gate_stride >= nq * DV && gate_stride % 4 == 0 && (uintptr_t)gate % 8 == 0)),
                "pico_attnb: gate rows must be 8-byte aligned and hold all heads");
   PICO_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "pico_attnb: chunks or a window, not both");
+  PICO_REQUIRE(out || (split && chunks > 1), "pico_attnb: without an output the pieces are left to the caller");
   PICO_REQUIRE(out_stride >= nq * DV && out_stride % 4 == 0 && (uintptr_t)out % (out_f32 ? 16 : 8) == 0,
                "pico_attnb: output rows of %d must hold all heads and start on four entries", out_stride);
   PICO_REQUIRE(v_div >= 1 && nkv % v_div == 0, "pico_attnb: %d kv heads do not share values %d each", nkv, v_div);
@@ -367,7 +368,7 @@ extern "C" int pico_attnb(const void* q, int q_stride, const void* k_cache, cons
              chunk, sink, gate_heads, v_div, out_f32, sinks, out_scale, out_stride};
   if (split) {
     attn_bias_kernel<true><<<dim3((unsigned)tiles, nkv, chunks), 256, 0, stream>>>(a);
-    if (chunks > 1)
+    if (chunks > 1 && out)                               // (no output: the caller puts the pieces together)
       attn_bias_merge_kernel<<<T * nq, DV <= 64 ? 64 : DV <= 128 ? 128 : 256, 0, stream>>>(parts_o, parts_ml, chunks, T * nq,
                                                                                            (bf16_t*)out, (const bf16_t*)gate,
                                                                                            gate_stride, nq, sink, gate_heads, out_f32, sinks,

@@ -85,9 +85,11 @@ class FastBiasAttention:
 
     def run(self, q: torch.Tensor, k_cache, v_cache, block_table, cu_seqlens, positions, num_seqs: int,
             split: Optional[bool] = None, out: Optional[torch.Tensor] = None, chunks: Optional[int] = None,
-            gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+            gate: Optional[torch.Tensor] = None, pieces: bool = False):
         """q [T, >= nq * dk] bfloat16 (row stride free); any mixture of portions and single tokens; returns [T, nq * dv].
-        ``gate`` [T, >= nq * dv] bfloat16 (8-byte aligned rows): the output is multiplied with sigmoid(gate)."""
+        ``gate`` [T, >= nq * dv] bfloat16 (8-byte aligned rows): the output is multiplied with sigmoid(gate).  ``pieces`` (keys
+        cut into several): returns (unnormalised sums [pieces, T nq, dv], their (maximum, sum) [pieces, T nq, 2]) instead, for a
+        launch that puts them together (with sink, gate and factor)."""
         T = q.shape[0]
         pages, P = _check_cache2(k_cache, v_cache, self.nkv, self.dk, self.dv, self.nkv // self.v_div)
         if not q.is_cuda or q.dtype != torch.bfloat16 or k_cache.dtype != torch.bfloat16:
@@ -107,7 +109,9 @@ class FastBiasAttention:
                                  or (not self.gate_heads and ((T > 1 and gate.stride(0) % 4) or gate.data_ptr() % 8))):
             raise KernelError("the gate must be bfloat16 [T, >= nq*dv] with unit stride along the row and 8-byte aligned rows")
         odt = torch.float32 if self.out_f32 else torch.bfloat16
-        if out is None:
+        if pieces:
+            out = None
+        elif out is None:
             out = torch.empty(T, self.nq * self.dv, dtype=odt, device=q.device)
         elif not out.is_cuda or tuple(out.shape) != (T, self.nq * self.dv) or out.dtype != odt or out.stride(1) != 1:
             raise KernelError("attention: out has the wrong shape or dtype")
@@ -115,6 +119,8 @@ class FastBiasAttention:
             split = self.split(T)
         if chunks is None:
             chunks = self.chunks(T, num_seqs) if split else 1
+        if pieces and (not split or chunks < 2):
+            raise KernelError("pieces are asked for where the keys are not cut")
         parts_o = parts_ml = None
         if chunks > 1:
             if not split:
@@ -128,8 +134,8 @@ class FastBiasAttention:
             1 if split else 0, chunks, _ptr(parts_o), _ptr(parts_ml), c_float(self.softcap), self.keep_first, _ptr(gate),
             0 if gate is None else (gate.stride(0) if T > 1 else gate.shape[1]), self.chunk, 1 if self.sink else 0,
             1 if self.gate_heads else 0, self.v_div, 1 if self.out_f32 else 0, _ptr(self.sinks), c_float(self.out_scale),
-            out.stride(0) if T > 1 else self.nq * self.dv, _stream()))
-        return out
+            out.stride(0) if T > 1 and out is not None else self.nq * self.dv, _stream()))
+        return (parts_o, parts_ml) if pieces else out
 
     def __call__(self, qkv, cache, block_table, ctx, gate=None, out=None):
         split, chunks, shape = self.plan(ctx)

@@ -915,6 +915,72 @@ def gated_row_norm(o: torch.Tensor, x: torch.Tensor, g_col: int, weight: torch.T
     return out
 
 
+# ---- two mixers side by side, a step of single tokens ----------------------------------------------------------------------
+PAIR_MAX_ROW, PAIR_MAX_PIECES = 4096, 64
+
+
+def pair_open(x: torch.Tensor, att: tuple, eps: float, cos_sin: Optional[torch.Tensor], rotary_dim: int, slots: torch.Tensor,
+              k_cache: torch.Tensor, v_cache: torch.Tensor, lin: tuple, state_slots: torch.Tensor, decay: torch.Tensor,
+              state: torch.Tensor):
+    """One launch for x bfloat16 [T, columns], a token a sequence.  ``att`` = (column of q, of k, of v, query heads, kv heads,
+    key size, value size): unit norm of every head of q and k, rotation of neighbours, store, as ``qk_norm_store``.
+    ``lin`` = (column of q, of k, of v, heads, key size, value size): S <- decay S + k v^T, o = S^T q with q, k, v through
+    z sigmoid(z), as ``gla_scan`` (``state`` updated in place).  Returns (the queries [T, nq * dk], o float32 [T, heads * dv])."""
+    _gpu(x, cos_sin, slots, k_cache, v_cache, state_slots, decay, state)
+    T = x.shape[0]
+    q_col, k_col, v_col, nq, nk, dk, dv = att
+    lq_col, lk_col, lv_col, heads, ldk, ldv = lin
+    if x.dtype != torch.bfloat16 or x.dim() != 2 or x.stride(1) != 1:
+        raise KernelError("pair_open: x must be bfloat16 [T, columns] with unit stride along the row")
+    if x.shape[1] < max(q_col + nq * dk, k_col + nk * dk, v_col + nk * dv, lq_col + heads * ldk, lk_col + heads * ldk, lv_col + heads * ldv):
+        raise KernelError("pair_open: the rows do not hold both sides")
+    pages, P = _check_cache2(k_cache, v_cache, nk, dk, dv)
+    if k_cache.dtype != torch.bfloat16:
+        raise KernelError("cache and activations differ in dtype")
+    if rotary_dim % 2 or not 0 <= rotary_dim <= dk:
+        raise KernelError(f"pair_open: {rotary_dim} turned entries do not fit a head of {dk}")
+    _check_table(cos_sin, T, rotary_dim // 2)
+    _i32(slots, "slots", T)
+    _i32(state_slots, "state_slots", T)
+    _vec(decay, heads, "the heads' decays")
+    if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, ldk, ldv) or not state.is_contiguous():
+        raise KernelError(f"pair_open: the state must be contiguous float32 [slots, {heads}, {ldk}, {ldv}]")
+    q = torch.empty(T, nq * dk, dtype=x.dtype, device=x.device)
+    o = torch.empty(T, heads * ldv, dtype=torch.float32, device=x.device)
+    lib = library.core()
+    _check(lib, lib.pico_pair_open(_ptr(x), x.stride(0) if T > 1 else x.shape[1], T, q_col, k_col, v_col, nq, nk, dk, dv, rotary_dim,
+                                   c_float(eps), _ptr(cos_sin) if rotary_dim else None, _ptr(slots), _ptr(q), _ptr(k_cache), _ptr(v_cache), P,
+                                   pages, lq_col, lk_col, lv_col, heads, ldk, ldv, _ptr(state_slots), _ptr(decay), _ptr(state), _ptr(o),
+                                   state.shape[0], _stream()))
+    return q, o
+
+
+def pair_close(parts_o: torch.Tensor, parts_ml: torch.Tensor, sinks: torch.Tensor, gate: torch.Tensor, out_scale: float,
+               out: torch.Tensor, o: torch.Tensor, lgate: torch.Tensor, weight: torch.Tensor, eps: float, lout: torch.Tensor) -> None:
+    """One launch: the pieces of an attention's keys (``FastBiasAttention.run(pieces=True)``) put together into ``out`` [T, nq *
+    dv] with the sinks' scores [nq], times sigmoid(``gate`` [T, >= nq]) and ``out_scale``; and the rows of ``o`` float32 [T, N]
+    RMS-normed with ``weight`` [N], times sigmoid(``lgate`` [T, >= N]), into ``lout`` [T, N].  Rows of outputs and gates may lie
+    in wider buffers."""
+    _gpu(parts_o, parts_ml, sinks, gate, out, o, lgate, weight, lout)
+    T, N = o.shape
+    nq = sinks.numel()
+    pieces, cols, dv = parts_o.shape
+    if parts_o.dtype != torch.float32 or parts_ml.dtype != torch.float32 or cols != T * nq or tuple(parts_ml.shape) != (pieces, cols, 2) \
+            or not parts_o.is_contiguous() or not parts_ml.is_contiguous():
+        raise KernelError("pair_close: the pieces must be contiguous float32 [pieces, T * nq, dv] and [pieces, T * nq, 2]")
+    _vec(sinks, nq, "the sinks' scores"); _vec(weight, N, "norm weight")
+    if o.dtype != torch.float32 or not o.is_contiguous():
+        raise KernelError("pair_close: o must be contiguous float32")
+    for t, n in ((gate, nq), (lgate, N), (out, nq * dv), (lout, N)):
+        if t.dtype != torch.bfloat16 or t.dim() != 2 or t.shape[0] != T or t.shape[1] < n or t.stride(1) != 1:
+            raise KernelError("pair_close: gates and outputs must be bfloat16 rows with unit stride")
+    st = lambda t: t.stride(0) if T > 1 else t.shape[1]
+    lib = library.core()
+    _check(lib, lib.pico_pair_close(T, _ptr(parts_o), _ptr(parts_ml), pieces, nq, dv, _ptr(sinks), _ptr(gate), st(gate), c_float(out_scale),
+                                    _ptr(out), st(out), _ptr(o), _ptr(lgate), st(lgate), N, _ptr(weight), c_float(eps), _ptr(lout), st(lout),
+                                    _stream()))
+
+
 MOE_MAX_TOP = 16
 
 

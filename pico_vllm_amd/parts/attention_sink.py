@@ -8,6 +8,7 @@ import torch
 from ..ops import kernels
 from .attention_bias import kv_page_tensors
 from .base import OpenMixer, StepContext
+from .lightning import LightningAttention
 from .registry import register_part
 from .rotary import PairsTable
 from .spec import CacheSpec, ParamSpec
@@ -96,3 +97,26 @@ class SinkAttention(OpenMixer):
             return
         kernels.attn_bias_plain(q, cache.k, cache.v, bt, ctx.positions, ctx.token_seq, self.nq, self.nkv, self.dk, self.dv, self.scale,
                                 self.window, gate=gate, gate_heads=True, sinks=self.sinks, out=out, out_scale=self.out_scale)
+
+    def core_beside(self, other: OpenMixer, y: torch.Tensor, col: int, other_col: int, ctx: StepContext, cache, other_cache,
+                    out: torch.Tensor, other_out: torch.Tensor) -> bool:
+        """This core and a ``LightningAttention``'s in shared launches, for a step of single tokens in bfloat16: norm, rotation
+        and store beside the walk of a token; attention over cut keys; the pieces put together beside the norm over all heads.
+        False: nothing was done (another mixer, another step, sizes that the launches do not take)."""
+        if not (isinstance(other, LightningAttention) and self.fast is not None and cache.k.dtype == torch.bfloat16 and ctx.all_decode
+                and ctx.num_tokens == ctx.num_seqs and other.heads * other.dv <= kernels.PAIR_MAX_ROW):
+            return False
+        split, pieces, shape = self.fast.plan(ctx)
+        if shape or not split or not 2 <= pieces <= kernels.PAIR_MAX_PIECES:
+            return False
+        table = self.angles.table(ctx) if self.angles is not None else None
+        q, o = kernels.pair_open(
+            y, (col, col + self.k_col, col + self.v_col, self.nq, self.nkv, self.dk, self.dv), self.norm_eps, table,
+            self.angles.rotary_dim if self.angles is not None else 0, ctx.slot_mapping[cache.group], cache.k, cache.v,
+            (other_col, other_col + other.k_col, other_col + other.v_col, other.heads, other.dk, other.dv), ctx.state_slots, other.decay,
+            other_cache.state)
+        parts = self.fast.run(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.positions, ctx.num_seqs, split=True,
+                              chunks=pieces, pieces=True)
+        kernels.pair_close(*parts, self.sinks, y[:, col + self.g_col:], self.out_scale, out, o, y[:, other_col + other.g_col:],
+                           other.norm_weight, other.norm_eps, other_out)
+        return True

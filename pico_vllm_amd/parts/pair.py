@@ -61,7 +61,8 @@ class MixerSum(Mixer):
     for, whose products are made together: ONE product makes the columns of both from h, both cores write side by side into
     one buffer (with the scales on what they write, in float32 in front of its rounding), and ONE product over that buffer is
     the sum.  Each side's columns start on eight entries (rows of zeros between them), so that what reads them may read
-    whole words.  ``left`` / ``right``: the two mixers as PartSpecs; their tensors stand behind ``prefixes``."""
+    whole words.  A left side with ``core_beside`` may run both cores in launches of its own (a step of single tokens, where
+    every launch is a chain of latencies).  ``left`` / ``right``: the two mixers as PartSpecs; their tensors stand behind ``prefixes``."""
 
     graph_safe_prompts = True
     ALIGN = 8
@@ -113,6 +114,9 @@ class MixerSum(Mixer):
         y = self.proj(x)
         whole = sum(self.out_cols) == self.out_total
         out = (torch.empty if whole else torch.zeros)(x.shape[0], self.out_total, dtype=x.dtype, device=x.device)
-        for part, own, i, c, n in zip(self.sides, cache, self.in_at, self.out_at, self.out_cols):
-            part.core(y, i, ctx, own, out[:, c:c + n])
+        outs = [out[:, c:c + n] for c, n in zip(self.out_at, self.out_cols)]
+        beside = getattr(self.left, "core_beside", None)
+        if beside is None or not beside(self.right, y, *self.in_at, ctx, *cache, *outs):
+            for part, own, i, o in zip(self.sides, cache, self.in_at, outs):
+                part.core(y, i, ctx, own, o)
         return self.o.partial(out)

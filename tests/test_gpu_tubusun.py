@@ -363,6 +363,59 @@ def test_the_norm_over_all_heads_and_its_gate(dtype, T, N):
     assert float((wide[:, :8].float() - 5).abs().max()) == 0 and float((wide[:, 8 + N:].float() - 5).abs().max()) == 0
 
 
+@pytest.mark.parametrize("H,G,dk,dv,rot,lh,ldk,ldv", [(6, 2, 64, 64, 32, 3, 64, 128), (3, 1, 24, 40, 10, 2, 9, 11), (20, 1, 32, 16, 0, 1, 200, 70), (2, 2, 7, 1, 6, 4, 1, 1),
+                                                      (4, 2, 160, 96, 160, 2, 130, 65)])
+def test_both_sides_of_a_step_of_single_tokens_in_one_launch(H, G, dk, dv, rot, lh, ldk, ldv):
+    from pico_vllm_amd.ops import kernels
+    g = torch.Generator().manual_seed(H * dk)
+    T, page, pages = 5, 8, 6
+    left_cols = (H + G) * dk + G * dv
+    at = -(-left_cols // 8) * 8
+    x = rounded(2 * torch.randn(T, at + 2 * lh * (ldk + ldv), generator=g, dtype=F), "bfloat16")
+    xd = x.to(DEV, torch.bfloat16)
+    i32 = lambda *v: torch.tensor(v, dtype=torch.int32, device=DEV)
+    slots, state_slots = i32(5, 11, -1, 47, 0), i32(2, 0, 3, 5, 1)
+    decay = [0.3, 0.99, 1.0, 0.8][:lh]
+    table = kernels.rope_table(i32(9, 70, 0, 300, 41), torch.tensor([100.0 ** (-2.0 * i / rot) for i in range(rot // 2)]).to(DEV)) if rot else None
+    caches = [(torch.zeros(pages, G, page, dk, dtype=torch.bfloat16, device=DEV), torch.zeros(pages, G, dv, page, dtype=torch.bfloat16, device=DEV)) for _ in range(2)]
+    s0 = torch.randn(5, lh, ldk, ldv, generator=g)           # the slot 5 of the fourth token does not exist
+    state = s0.to(DEV)
+    q, o = kernels.pair_open(xd, (0, H * dk, (H + G) * dk, H, G, dk, dv), 1e-3, table, rot, slots, *caches[0],
+                             (at, at + lh * ldk, at + 2 * lh * ldk, lh, ldk, ldv), state_slots, torch.tensor(decay, device=DEV), state)
+    q2 = kernels.qk_norm_store(xd, 0, H * dk, (H + G) * dk, H, G, G, dk, dv, 1, kernels.QK_NORM_UNIT, None, None, 1e-3, table, rot, slots, *caches[1], pairs=True)
+    close(q, q2, "bfloat16", scale=0.3)
+    close(caches[0][0], caches[1][0].double(), "bfloat16", scale=0.3)
+    assert torch.equal(caches[0][1], caches[1][1])
+    for t, slot in enumerate(state_slots.tolist()):
+        if slot < 5:
+            want, last = lightning_plain(x[t:t + 1, at:], lh, ldk, ldv, [float(d) for d in torch.tensor(decay)], s0[slot].to(F))
+            close(o[t].view(lh, ldv), want[0], "float32", scale=2)
+            close(state[slot], last, "float32", scale=2)
+    assert torch.equal(state[4].cpu(), s0[4])
+
+
+@pytest.mark.parametrize("T,H,dv,pieces,N", [(1, 6, 64, 7, 384), (5, 3, 40, 2, 22), (9, 20, 16, 64, 4096), (2, 1, 256, 33, 1), (3, 5, 1, 3, 1025)])
+def test_pieces_put_together_beside_the_norm_over_all_heads(T, H, dv, pieces, N):
+    from pico_vllm_amd.ops import kernels
+    g = torch.Generator().manual_seed(T * H + N)
+    po, mx, l = torch.randn(pieces, T * H, dv, generator=g), 5 * torch.randn(pieces, T * H, generator=g), 1 + torch.rand(pieces, T * H, generator=g)
+    if pieces > 2:
+        mx[1, ::2], l[1, ::2], po[1, ::2] = -float("inf"), 0.0, 0.0      # a piece in which a column saw no key
+    sinks = torch.tensor([1.0, 500.0, -30.0, 4.0] * 5)[:H]
+    gate, lgate = (rounded(torch.randn(T, n + 5, generator=g, dtype=F), "bfloat16") for n in (H, N))
+    o, w = torch.randn(T, N, generator=g), 1 + 0.3 * torch.randn(N, generator=g)
+    out, lout = (torch.full((T, n + 8), 5.0, dtype=torch.bfloat16, device=DEV) for n in (H * dv, N))
+    bf = lambda t: t.to(DEV, torch.bfloat16)
+    kernels.pair_close(po.to(DEV), torch.stack([mx, l], -1).to(DEV), sinks.to(DEV), bf(gate)[:, 2:], 0.7, out[:, 3:3 + H * dv], o.to(DEV), bf(lgate)[:, 1:],
+                       w.to(DEV), 1e-3, lout[:, 8:])
+    e = torch.exp(mx.to(F))
+    den = (e * l.to(F)).sum(0).view(T, H) + torch.exp(sinks.to(F))
+    want = (e[..., None] * po.to(F)).sum(0).view(T, H, dv) / den[..., None] * torch.sigmoid(gate[:, 2:2 + H])[..., None] * 0.7
+    close(out[:, 3:3 + H * dv], want.reshape(T, H * dv), "bfloat16")
+    close(lout[:, 8:], P.rms(o.to(F), 1e-3) * w.to(F) * torch.sigmoid(lgate[:, 1:1 + N]), "bfloat16")
+    assert all(float((v.float() - 5).abs().max()) == 0 for v in (out[:, :3], out[:, 3 + H * dv:], lout[:, :8]))
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("E,top,groups,keep,D", [(8, 2, 4, 2, 64), (16, 4, 4, 3, 128), (9, 3, 3, 2, 72), (5, 1, 1, 1, 44), (4, 2, 4, 2, 40), (160, 8, 8, 3, 96),
                                                  (12, 5, 2, 2, 50), (256, 16, 64, 5, 64), (130, 6, 130, 9, 32)])
