@@ -8,8 +8,8 @@
                                                              continuous batching with prompts cut into portions)
 
   python bench.py --workload designs --layers 4             (Lerazen and Nasedra, each beside the Qwen2.5 shape of equal size,
-                                                             Dikolix and Vagelix beside Nasedra, and Begasun beside Dikolix, at two
-                                                             sizes: decode at batch 1 and 8, the 2,048-token prefill;
+                                                             Dikolix and Vagelix beside Nasedra, Begasun beside Dikolix, Tubusun beside
+                                                             Vagelix, at two sizes: decode at batch 1 and 8, the 2,048-token prefill;
                                                              --designs nasedra measures that design's pairs only)
 
   python bench.py --workload long --shape 32b --device-weights --context 32768
